@@ -52,8 +52,6 @@ struct QAbsArgs;
 int kx_gemv_absorb_launch(KxGemvArgs g, const QAbsArgs &q, bool *fused, hipStream_t st);
 int kx_rmsnorm_launch(const uint16_t *x, const uint16_t *w, uint16_t *y, int tokens, int n, int x_stride,
                       int y_stride, float eps, hipStream_t st);
-int kx_argmax_launch(const float *logits, int tokens, int n, int stride, uint32_t *out, float *scratch, hipStream_t st);
-#define KX_ARGMAX_SCRATCH_FLOATS(tokens) ((size_t)(tokens) * 128)
 
 // kx_i4.hip
 // What the routed down launch needs to finish the MoE layer itself (up to 4 tokens): its workgroups and those of the

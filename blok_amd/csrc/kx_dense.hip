@@ -16,6 +16,7 @@
 #include <mutex>
 #include "kx_arrive.h"
 #include "kx_attn_parts.h"
+#include "kx_argmax.h"
 #include "kx_common.h"
 #include "kx_dense.h"
 #include "kx_gemv_body.h"
@@ -198,50 +199,6 @@ __global__ void __launch_bounds__(TT > 1 ? 512 : 1024) gemv_absorb_k(KxGemvArgs 
   if (threadIdx.x == 0) kx_arrive_reset(q.head_count + h);
 }
 
-// lowest-index argmax over bf16-rounded logits (sample_lm_head :718-734, argmax_k :477-493), in two
-// stages: ARGMAX_PARTS workgroups per row each reduce a slice, then one wave per row merges them
-constexpr int ARGMAX_PARTS = 64;
-
-__device__ __forceinline__ void argmax_merge(float &best, uint32_t &bi, float ov, uint32_t oi) {
-  if (ov > best || (ov == best && oi < bi)) { best = ov; bi = oi; }
-}
-__device__ __forceinline__ void argmax_wave(float &best, uint32_t &bi) {
-  for (int m = 32; m; m >>= 1) {
-    float ov = __shfl_xor(best, m);
-    uint32_t oi = (uint32_t)__shfl_xor((int)bi, m);
-    argmax_merge(best, bi, ov, oi);
-  }
-}
-
-__global__ void __launch_bounds__(256) argmax_part_k(const float *__restrict__ logits, int n, int stride,
-                                                     float *__restrict__ pv, uint32_t *__restrict__ pi) {
-  __shared__ float sv[4];
-  __shared__ uint32_t si[4];
-  const float *p = logits + (size_t)blockIdx.y * stride;
-  const int per = (n + ARGMAX_PARTS - 1) / ARGMAX_PARTS;
-  const int lo = blockIdx.x * per, hi = min(n, lo + per);
-  float best = -__builtin_inff();
-  uint32_t bi = 0xffffffffu;
-  for (int i = lo + threadIdx.x; i < hi; i += blockDim.x) {
-    float v = p[i];
-    if (v > best) { best = v; bi = (uint32_t)i; }
-  }
-  argmax_wave(best, bi);
-  if ((threadIdx.x & 63) == 0) { sv[threadIdx.x >> 6] = best; si[threadIdx.x >> 6] = bi; }
-  __syncthreads();
-  if (threadIdx.x == 0) {
-    for (int w = 1; w < 4; ++w) argmax_merge(best, bi, sv[w], si[w]);
-    pv[blockIdx.y * ARGMAX_PARTS + blockIdx.x] = best;
-    pi[blockIdx.y * ARGMAX_PARTS + blockIdx.x] = bi;
-  }
-}
-__global__ void __launch_bounds__(64) argmax_final_k(const float *__restrict__ pv, const uint32_t *__restrict__ pi,
-                                                     uint32_t *__restrict__ out) {
-  float best = pv[blockIdx.x * ARGMAX_PARTS + threadIdx.x];
-  uint32_t bi = pi[blockIdx.x * ARGMAX_PARTS + threadIdx.x];
-  argmax_wave(best, bi);
-  if (threadIdx.x == 0) out[blockIdx.x] = bi == 0xffffffffu ? 0u : bi;  // every logit -inf or NaN: id 0 as :481
-}
 
 template <int MATS, int RI>
 void launch_tt(const KxGemvArgs &a, int tt, dim3 g, dim3 b, size_t lds, hipStream_t st) {
@@ -515,17 +472,6 @@ int kx_rmsnorm_launch(const uint16_t *x, const uint16_t *w, uint16_t *y, int tok
   return KX_OK;
 }
 
-// scratch: tokens * ARGMAX_PARTS floats and as many uint32
-int kx_argmax_launch(const float *logits, int tokens, int n, int stride, uint32_t *out, float *scratch, hipStream_t st) {
-  float *pv = scratch;
-  uint32_t *pi = (uint32_t *)(scratch + (size_t)tokens * ARGMAX_PARTS);
-  hipLaunchKernelGGL(argmax_part_k, dim3(ARGMAX_PARTS, tokens), dim3(256), 0, st, logits, n, stride, pv, pi);
-  KX_LAUNCH_CHECK();
-  hipLaunchKernelGGL(argmax_final_k, dim3(tokens), dim3(64), 0, st, pv, pi, out);
-  KX_LAUNCH_CHECK();
-  return KX_OK;
-}
-
 extern "C" int kx_rmsnorm(const void *d_x, const void *d_w, void *d_y, int32_t tokens, int32_t n, float eps,
                           void *stream) {
   KX_REQUIRE(d_x && d_w && d_y, "kx_rmsnorm: null pointer");
@@ -547,12 +493,12 @@ extern "C" int kx_lm_head_argmax(const void *d_w, const void *d_n, void *d_logit
 }
 
 // ---- the same operator for callers that may not allocate ---------------------------------------
-// The per-token argmax partials (ARGMAX_PARTS values and indices per token) live in a file-scope device
+// The per-token argmax partials (KX_ARGMAX_PARTS values and indices per token) live in a file-scope device
 // array instead of a caller's buffer.  Every GPU holds its own copy of the array at its own address, so
 // the address is looked up once per device, with that device current, and kept.
 constexpr int KX_STATIC_ARGMAX_TOKENS = 256;
 constexpr int KX_STATIC_MAX_DEVICES = 64;
-static __device__ __align__(256) unsigned char g_argmax_scratch[KX_STATIC_ARGMAX_TOKENS * ARGMAX_PARTS * 8];
+static __device__ __align__(256) unsigned char g_argmax_scratch[KX_STATIC_ARGMAX_TOKENS * KX_ARGMAX_PARTS * 8];
 static std::mutex g_argmax_scratch_mu;
 static void *g_argmax_scratch_ptr[KX_STATIC_MAX_DEVICES];
 

@@ -1,0 +1,526 @@
+// kx_hybrid.hip -- the hybrid decoder: weights, cache and state, one step of the stack, and its entry in the registry.
+// The loops around a step -- prefill, decode, sampling -- are kx_stack.hip's, as for the other design.
+//
+// A step of T tokens (T = positions x sequences), per layer:
+//   all input projections of the mixer as one product, the streams' read-out and the norm in front of it
+//   -> attention over window and pooled blocks (kx_window.hip), or convolutions and delta rule (kx_delta.hip)
+//   -> output projection; its epilogue updates all residual streams
+//   -> gate and up as one product with the clamped activation, norm in front -> down, which updates the streams.
+// Up to 4 tokens the products are GEMVs that build their activation rows themselves (kx_linear.hip).
+// The residual streams, the projections a mixer reads, scores, recurrent state and convolution inputs are 32-bit in
+// both number formats; bf16 are weights, activation rows of the products and the key/value cache.
+#include <string.h>
+#include <algorithm>
+#include <vector>
+#include "kx_argmax.h"
+#include "kx_hybrid.h"
+#include "kx_linear.h"
+#include "kx_load.h"
+#include "kx_math.h"
+#include "kx_model.h"
+#include "kx_safetensors.h"
+
+namespace {
+
+// one tensor of the files and where it goes
+struct Slot {
+  std::string name;
+  int rows = 0, cols = 0;  // cols 0: one dimension
+  void *dst = nullptr;
+  int ld = 0;      // matrices: elements per row of the arena; 0: an array of floats
+  int half = -1;   // 0, 1: gate, up rows of KX_GLU_BLOCK blocks
+  float mean = 0, sigma = 0;  // random init
+  size_t count() const { return (size_t)rows * (cols ? cols : 1); }
+};
+
+struct HyperW {
+  float *in = nullptr, *mix = nullptr, *out = nullptr;
+};
+struct LayerW {
+  float *norm1 = nullptr, *norm2 = nullptr;
+  HyperW hc[2];
+  KxMat in, o, gu, down;  // mixer projections back to back; output; gate and up; down
+  int q_off = 0, k_off = 0, v_off = 0, g_off = 0, b_off = 0, a_off = 0;  // rows of `in`
+  float *q_norm = nullptr, *k_norm = nullptr;
+  float *conv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *o_norm = nullptr;
+  KxWindowCache cache;
+  float *state = nullptr, *hist[2] = {nullptr, nullptr};
+  size_t state_floats = 0, hist_floats = 0;  // per sequence
+};
+
+struct HybridModel : kx_model {
+  KxHybridConfig c;
+  std::string name;
+  bool f32 = false;
+  std::vector<LayerW> L;
+  KxMat embed, head;
+  float *final_norm = nullptr;
+  std::vector<Slot> slots;
+  float *streams = nullptr, *proj = nullptr, *delta_o = nullptr, *work = nullptr, *part = nullptr;
+  void *rows = nullptr, *att = nullptr, *q = nullptr, *mid = nullptr;
+  int proj_ld = 0, att_ld = 0, mid_ld = 0, part_tokens = 0;
+  size_t part_floats = 0;
+  int *want = nullptr;           // token rows of row_logits
+  float init_sigma_ = 0;
+  int hist_cur = 0;              // which of the two convolution histories the next step reads
+  float *record = nullptr;       // [n_layers][max_context][max_batch][width]
+
+  const char *design() const override { return name.c_str(); }
+  int step(const uint32_t *d_ids, bool sample, int C) override;
+  int step_positions(int batch_) const override { return std::max(1, step_tokens / batch_); }
+  int restart(int batch_) override;
+  int row_logits(const int *token_rows, int n, float *d_out) override;
+  int logit_rows() const override { return std::max(max_batch, 64); }
+  int rewind(int positions) override {
+    kx_set_error("kx_model_rewind: %s keeps recurrent state, which does not go back", design());
+    return KX_ERR_ARG;
+  }
+  int hidden_bf16(uint16_t *h_out) override;
+  int set_residual_record(bool on) override;
+  int residual(int layer, int pos0, int n, float *h_out) override;
+  ~HybridModel() override {
+    if (record) (void)hipFree(record);
+  }
+  size_t layout(char *base);
+  int fill(const std::string &dir, const kx_open_options &o);
+  int pack(const Slot &s, const void *src, bool src_f32);
+  int logits_of(const float *x, const int *map, int n, float *d_out);
+};
+
+// ---- kernels ----
+template <class T>
+__global__ void __launch_bounds__(256) pack_k(const void *src, int src_f32, T *dst, int rows, int cols, int ld, int half) {
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= (size_t)rows * cols) return;
+  const int r = (int)(i / cols), col = (int)(i - (size_t)r * cols);
+  const float v = src_f32 ? ((const float *)src)[i] : kx_bf16_f32(((const uint16_t *)src)[i]);
+  const int to = half < 0 ? r : (r / KX_GLU_BLOCK) * 2 * KX_GLU_BLOCK + r % KX_GLU_BLOCK + half * KX_GLU_BLOCK;
+  if constexpr (sizeof(T) == 4) dst[(size_t)to * ld + col] = v;
+  else dst[(size_t)to * ld + col] = kx_bf16_rne(v);
+}
+template <class T>
+__global__ void __launch_bounds__(256) embed_streams_k(const T *__restrict__ embed, int ld, const uint32_t *__restrict__ ids, float *__restrict__ x, int width,
+                                                       int streams) {
+  const T *e = embed + (size_t)ids[blockIdx.x] * ld;
+  float *o = x + (size_t)blockIdx.x * streams * width;
+  for (int c = threadIdx.x; c < width; c += 256) {
+    float v;
+    if constexpr (sizeof(T) == 4) v = e[c];
+    else v = kx_bf16_f32(e[c]);
+    for (int s = 0; s < streams; ++s) o[(size_t)s * width + c] = v;
+  }
+}
+// sum of the streams of token blockIdx.x into row (blockIdx.x / nb) * stride + blockIdx.x % nb of out
+__global__ void __launch_bounds__(256) sum_streams_k(const float *__restrict__ x, float *__restrict__ out, int width, int streams, int nb, int stride) {
+  const int t = blockIdx.x;
+  const float *p = x + (size_t)t * streams * width;
+  float *o = out + ((size_t)(t / nb) * stride + t % nb) * width;
+  for (int c = threadIdx.x; c < width; c += 256) {
+    float v = p[c];
+    for (int s = 1; s < streams; ++s) v += p[(size_t)s * width + c];
+    o[c] = v;
+  }
+}
+
+#define KX_TRY(call) do { if (int rc_ = (call)) return rc_; } while (0)
+
+// Lays everything out from `base` on (nullptr: sizes only) and lists the tensors the files have to hold.
+size_t HybridModel::layout(char *base) {
+  KxPlan p;
+  slots.clear();
+  L.assign(c.layers.size(), LayerW());
+  const size_t es = f32 ? 4 : 2;
+  const int S = c.streams, W = c.width;
+  auto at = [&](size_t bytes) -> char * {
+    const size_t off = p.take(bytes);
+    return base ? base + off : nullptr;
+  };
+  auto vec = [&](const std::string &n, int rows, int cols, float mean, float sigma) {
+    Slot s;
+    s.name = n; s.rows = rows; s.cols = cols; s.mean = mean; s.sigma = sigma;
+    s.dst = at(s.count() * 4);
+    slots.push_back(s);
+    return (float *)s.dst;
+  };
+  auto mat = [&](int rows, int cols) {
+    KxMat m;
+    m.rows = rows; m.cols = cols; m.ld = kx_pad(cols, KX_LD);
+    m.w = at((size_t)rows * m.ld * es);
+    return m;
+  };
+  const float sg = init_sigma_;
+  auto part_of = [&](const KxMat &m, int row0, const std::string &n, int rows, int half, float sigma) {
+    Slot s;
+    s.name = n; s.rows = rows; s.cols = m.cols; s.ld = m.ld; s.half = half; s.sigma = sigma;
+    s.dst = m.w ? (char *)m.w + (size_t)row0 * m.ld * es : nullptr;
+    slots.push_back(s);
+  };
+  embed = mat(c.vocab, W);
+  part_of(embed, 0, "embed", c.vocab, -1, 1.0f);
+  int row_ld = kx_pad(W, KX_LD);
+  proj_ld = att_ld = mid_ld = 0;
+  size_t q_cols = 0, o_cols = 0, work_floats = 0;
+  part_floats = 0;
+  for (size_t i = 0; i < c.layers.size(); ++i) {
+    const KxHybridLayer &l = c.layers[i];
+    LayerW &w = L[i];
+    const std::string n = "l" + std::to_string(i) + ".", m = n + "mix.";
+    auto hyper = [&](int q) {
+      HyperW h;
+      if (!c.hyper) return h;
+      const std::string k = n + "hc" + std::to_string(q) + ".";
+      h.in = vec(k + "in", S, 0, 1.0f / S, 0.02f);
+      h.out = vec(k + "out", S, 0, 1.0f, 0.02f);
+      h.mix = vec(k + "mix", S, S, 1.0f / S, 0.02f);
+      return h;
+    };
+    w.norm1 = vec(n + "norm1", W, 0, 1.0f, 0.02f);
+    w.hc[0] = hyper(1);
+    // the mixer's projections, each from a multiple of 32 rows on
+    struct Piece { const char *name; int rows; int *off; };
+    std::vector<Piece> pieces;
+    const bool attn = l.mixer == KxHybridLayer::ATTENTION;
+    const int out_cols = attn ? l.attn.heads * l.attn.vdim : l.delta.heads * l.delta.vdim;
+    if (attn) {
+      pieces = {{"q", l.attn.heads * l.attn.dim, &w.q_off}, {"k", l.attn.kv_heads * l.attn.dim, &w.k_off}, {"v", l.attn.kv_heads * l.attn.vdim, &w.v_off}};
+      if (l.gate) pieces.push_back({"g", out_cols, &w.g_off});
+    } else {
+      pieces = {{"q", l.delta.kv_heads * l.delta.dim, &w.q_off}, {"k", l.delta.kv_heads * l.delta.dim, &w.k_off}, {"v", out_cols, &w.v_off},
+                {"g", out_cols, &w.g_off}, {"b", l.delta.heads, &w.b_off}, {"a", l.delta.heads, &w.a_off}};
+    }
+    int rows_in = 0;
+    for (const Piece &x : pieces) {
+      *x.off = rows_in;
+      rows_in += kx_pad(x.rows, 32);
+    }
+    w.in = mat(rows_in, W);
+    for (const Piece &x : pieces) part_of(w.in, *x.off, m + x.name, x.rows, -1, sg);
+    w.o = mat(W, out_cols);
+    part_of(w.o, 0, m + "o", W, -1, sg);
+    proj_ld = std::max(proj_ld, rows_in);
+    row_ld = std::max(row_ld, w.o.ld);
+    if (attn) {
+      if (l.qk_norm) {
+        w.q_norm = vec(m + "q.norm", l.attn.heads * l.attn.dim, 0, 1.0f, 0.02f);
+        w.k_norm = vec(m + "k.norm", l.attn.kv_heads * l.attn.dim, 0, 1.0f, 0.02f);
+      }
+      att_ld = std::max(att_ld, w.o.ld);
+      q_cols = std::max(q_cols, (size_t)l.attn.heads * kx_pad(l.attn.dim, 32));
+      part_floats = std::max(part_floats, kx_window_part_floats(l.attn, max_context, part_tokens));
+    } else {
+      const KxDeltaSpec &d = l.delta;
+      const int C = kx_delta_channels(d), nq = d.kv_heads * d.dim;
+      w.conv = (float *)at((size_t)C * d.taps * 4);  // q, k and v channels back to back
+      int ch = 0;
+      for (const Piece &x : {Piece{"q.conv", nq, nullptr}, Piece{"k.conv", nq, nullptr}, Piece{"v.conv", out_cols, nullptr}}) {
+        Slot s;
+        s.name = m + x.name; s.rows = x.rows; s.cols = d.taps; s.sigma = 0.5f;
+        s.dst = w.conv ? w.conv + (size_t)ch * d.taps : nullptr;
+        slots.push_back(s);
+        ch += x.rows;
+      }
+      w.a_log = vec(m + "A_log", d.heads, 0, 0.0f, 0.5f);
+      w.dt_bias = vec(m + "dt_bias", d.heads, 0, -2.0f, 0.5f);
+      w.o_norm = vec(m + "norm", d.vdim, 0, 1.0f, 0.02f);
+      o_cols = std::max(o_cols, (size_t)out_cols);
+      work_floats = std::max(work_floats, kx_delta_work_floats(d));
+      w.state_floats = (size_t)d.heads * d.dim * d.vdim;
+      w.hist_floats = (size_t)(d.taps - 1) * C;
+    }
+    if (l.ff) {
+      w.norm2 = vec(n + "norm2", W, 0, 1.0f, 0.02f);
+      w.hc[1] = hyper(2);
+      w.gu = mat(2 * kx_pad(l.ff, KX_GLU_BLOCK), W);
+      part_of(w.gu, 0, n + "mlp.gate", l.ff, 0, sg);
+      part_of(w.gu, 0, n + "mlp.up", l.ff, 1, sg);
+      w.down = mat(W, l.ff);
+      part_of(w.down, 0, n + "mlp.down", W, -1, sg);
+      mid_ld = std::max(mid_ld, w.down.ld);
+    }
+  }
+  final_norm = vec("final.norm", W, 0, 1.0f, 0.02f);
+  head = mat(c.vocab, W);
+  part_of(head, 0, "head", c.vocab, -1, sg);
+  weight_bytes = p.total;
+
+  for (size_t i = 0; i < c.layers.size(); ++i) {
+    const KxHybridLayer &l = c.layers[i];
+    LayerW &w = L[i];
+    if (l.mixer == KxHybridLayer::ATTENTION) {
+      size_t e[4];
+      kx_window_shape(l.attn, max_context, std::min(step_tokens, max_context), &w.cache, e);
+      w.cache.k = at(e[0] * max_batch * es);
+      w.cache.v = at(e[1] * max_batch * es);
+      w.cache.pk = at(e[2] * max_batch * es);
+      w.cache.pv = at(e[3] * max_batch * es);
+    } else {
+      w.state = (float *)at(w.state_floats * max_batch * 4);
+      for (auto &h : w.hist) h = (float *)at(w.hist_floats * max_batch * 4);
+    }
+  }
+  cache_bytes = p.total - weight_bytes;
+
+  const size_t T = step_tokens, B = max_batch;
+  streams = (float *)at(T * S * W * 4);
+  proj = (float *)at(T * proj_ld * 4);
+  delta_o = (float *)at(T * o_cols * 4);
+  work = (float *)at(T * work_floats * 4);
+  part = (float *)at(part_floats * 4);
+  rows = at(std::max(T, (size_t)logit_rows()) * row_ld * es);
+  att = at(T * att_ld * es);
+  q = at(T * q_cols * es);
+  mid = at(T * mid_ld * es);
+  logits = (float *)at((size_t)logit_rows() * c.vocab * 4);
+  argmax_scratch = (float *)at(KX_ARGMAX_SCRATCH_FLOATS(B) * 4);
+  ids = (uint32_t *)at((size_t)max_context * B * 4);
+  next = (uint32_t *)at(B * 4);
+  history = (uint32_t *)at((size_t)max_context * B * 4);
+  want = (int *)at((size_t)logit_rows() * 4);
+  scratch_bytes = p.total - weight_bytes - cache_bytes;
+  return p.total;
+}
+
+int HybridModel::pack(const Slot &s, const void *src, bool src_f32) {
+  const int rows_ = s.rows, cols = s.cols ? s.cols : 1, ld = s.ld ? s.ld : cols;
+  const dim3 grid((unsigned)((s.count() + 255) / 256));
+  if (f32 || !s.ld) hipLaunchKernelGGL(pack_k<float>, grid, dim3(256), 0, st, src, src_f32, (float *)s.dst, rows_, cols, ld, s.half);
+  else hipLaunchKernelGGL(pack_k<uint16_t>, grid, dim3(256), 0, st, src, src_f32, (uint16_t *)s.dst, rows_, cols, ld, s.half);
+  KX_LAUNCH_CHECK();
+  return KX_OK;
+}
+
+struct Staging {  // device memory that is gone at the end of a scope
+  char *p = nullptr;
+  ~Staging() { if (p) (void)hipFree(p); }
+};
+
+// The tensors from the files (or from the generator), through a staging buffer: the files have rows without padding,
+// gate and up apart, and bf16 where the arena may have f32.
+int HybridModel::fill(const std::string &dir, const kx_open_options &o) {
+  constexpr size_t BATCH = (size_t)1 << 30;
+  KxTensorMap files;
+  if (!o.random_init) {
+    KX_TRY(kx_safetensors_scan(dir, files));
+    for (const Slot &s : slots) {
+      const auto f = files.find(s.name);
+      KX_REQUIRE(f != files.end(), "missing tensor: %s (%s)", s.name.c_str(), dir.c_str());
+      const std::string shape = std::to_string(s.rows) + (s.cols ? "x" + std::to_string(s.cols) : "");
+      KX_REQUIRE(f->second.shape == shape && f->second.dtype != "i32", "tensor %s is %s %s, expected bf16 or f32 %s", s.name.c_str(), f->second.dtype.c_str(),
+                 f->second.shape.c_str(), shape.c_str());
+    }
+  }
+  auto bytes_of = [&](const Slot &s) { return ((o.random_init ? s.count() * 2 : files.at(s.name).data_bytes) + 255) & ~(size_t)255; };
+  size_t most = 0;
+  for (size_t i = 0; i < slots.size();) {  // the largest batch
+    size_t sum = bytes_of(slots[i]), j = i + 1;
+    while (j < slots.size() && sum + bytes_of(slots[j]) <= BATCH) sum += bytes_of(slots[j++]);
+    most = std::max(most, sum);
+    i = j;
+  }
+  Staging stage;
+  KX_HIP(hipMalloc((void **)&stage.p, most));
+  for (size_t i = 0; i < slots.size();) {
+    std::vector<KxLoadItem> items;
+    size_t sum = 0, j = i;
+    for (; j < slots.size() && (j == i || sum + bytes_of(slots[j]) <= BATCH); ++j) {
+      if (o.random_init) KX_TRY(kx_fill_affine_bf16(stage.p + sum, slots[j].count(), o.seed, 1 + j, slots[j].mean, slots[j].sigma, st));
+      else items.push_back(KxLoadItem{&files.at(slots[j].name), stage.p + sum, false});
+      sum += bytes_of(slots[j]);
+    }
+    uint64_t bytes = 0;
+    double seconds = 0;
+    if (!o.random_init) KX_TRY(kx_load_run(items, &bytes, &seconds));
+    load_bytes += bytes;
+    load_seconds += seconds;
+    sum = 0;
+    for (; i < j; ++i) {
+      KX_TRY(pack(slots[i], stage.p + sum, !o.random_init && files.at(slots[i].name).dtype == "f32"));
+      sum += bytes_of(slots[i]);
+    }
+    KX_HIP(hipStreamSynchronize(st));  // the buffer is used again
+  }
+  return KX_OK;
+}
+
+int HybridModel::restart(int batch_) {
+  for (const LayerW &w : L) {
+    if (w.state) KX_HIP(hipMemsetAsync(w.state, 0, w.state_floats * batch_ * 4, st));
+    if (w.hist_floats) KX_HIP(hipMemsetAsync(w.hist[hist_cur], 0, w.hist_floats * batch_ * 4, st));
+  }
+  return KX_OK;
+}
+
+int HybridModel::logits_of(const float *x, const int *map, int n, float *d_out) {
+  KxLinArgs g;
+  g.m = head;
+  g.tokens = n;
+  g.row.kind = KX_ROW_NORM; g.row.cols = c.width; g.row.rows_map = map; g.row.streams = x; g.row.n_streams = c.streams; g.row.groups = c.groups;
+  g.row.w = final_norm; g.row.eps = c.eps;
+  g.out = d_out;
+  g.out_ld = c.vocab;
+  return kx_linear(f32, g, rows, st);
+}
+
+int HybridModel::step(const uint32_t *d_ids, bool sample, int C) {
+  const int T = batch * C, S = c.streams, W = c.width;
+  KX_REQUIRE(T > 0 && T <= std::max(step_tokens, max_batch), "%s: a step of %d tokens, at most %d", design(), T, step_tokens);
+  if (f32) hipLaunchKernelGGL(embed_streams_k<float>, dim3(T), dim3(256), 0, st, (const float *)embed.w, embed.ld, d_ids, streams, W, S);
+  else hipLaunchKernelGGL(embed_streams_k<uint16_t>, dim3(T), dim3(256), 0, st, (const uint16_t *)embed.w, embed.ld, d_ids, streams, W, S);
+  KX_LAUNCH_CHECK();
+  for (int i = 0; i < n_layers; ++i) {
+    const KxHybridLayer &l = c.layers[i];
+    LayerW &w = L[i];
+    auto read = [&](KxLinArgs &g, const KxMat &m, const float *norm, const HyperW &h) {  // norm(sum_s in[s] x_s) in front of m
+      g.m = m;
+      g.tokens = T;
+      g.row.kind = KX_ROW_NORM; g.row.cols = W; g.row.streams = streams; g.row.n_streams = S; g.row.in = h.in; g.row.groups = c.groups;
+      g.row.w = norm; g.row.eps = c.eps;
+    };
+    auto write = [&](KxLinArgs &g, const KxMat &m, const HyperW &h) {  // the product into the streams
+      g.m = m;
+      g.tokens = T;
+      g.row.cols = m.cols;
+      g.epi = KX_LIN_STREAMS;
+      g.streams = streams; g.n_streams = S; g.mix = h.mix; g.outw = h.out;
+    };
+    KxLinArgs in, out;
+    read(in, w.in, w.norm1, w.hc[0]);
+    in.out = proj;
+    in.out_ld = proj_ld;
+    KX_TRY(kx_linear(f32, in, rows, st));
+    write(out, w.o, w.hc[0]);
+    if (l.mixer == KxHybridLayer::ATTENTION) {
+      KxWindowArgs a;
+      a.s = l.attn; a.c = w.cache;
+      a.proj = proj; a.proj_ld = proj_ld; a.q_off = w.q_off; a.k_off = w.k_off; a.v_off = w.v_off; a.g_off = l.gate ? w.g_off : -1;
+      a.q_norm = w.q_norm; a.k_norm = w.k_norm; a.eps = c.eps;
+      a.batch = batch; a.positions = C; a.pos = pos;
+      a.out = att; a.out_ld = att_ld; a.q = q; a.part = part; a.part_floats = part_floats;
+      KX_TRY(kx_window_attention(f32, a, st));
+      out.row.x = att;
+      out.row.x_ld = att_ld;
+    } else {
+      KxDeltaArgs d;
+      d.s = l.delta;
+      d.proj = proj; d.proj_ld = proj_ld; d.q_off = w.q_off; d.k_off = w.k_off; d.v_off = w.v_off; d.b_off = w.b_off; d.a_off = w.a_off;
+      d.conv = w.conv; d.a_log = w.a_log; d.dt_bias = w.dt_bias;
+      d.state = w.state; d.hist = w.hist[hist_cur]; d.hist_out = w.hist[hist_cur ^ 1];
+      d.batch = batch; d.positions = C;
+      d.o = delta_o; d.work = work;
+      KX_TRY(kx_delta(d, st));
+      out.row.kind = KX_ROW_GATED;
+      out.row.o = delta_o; out.row.gate = proj + w.g_off; out.row.gate_ld = proj_ld; out.row.heads = l.delta.heads; out.row.vdim = l.delta.vdim;
+      out.row.w = w.o_norm; out.row.eps = c.eps;
+    }
+    KX_TRY(kx_linear(f32, out, rows, st));
+    if (l.ff) {
+      KxLinArgs gu, down;
+      read(gu, w.gu, w.norm2, w.hc[1]);
+      gu.epi = KX_LIN_GLU;
+      gu.mid = mid; gu.mid_ld = mid_ld; gu.limit = l.limit; gu.alpha = l.alpha; gu.bias = l.bias;
+      KX_TRY(kx_linear(f32, gu, rows, st));
+      write(down, w.down, w.hc[1]);
+      down.row.x = mid;
+      down.row.x_ld = mid_ld;
+      KX_TRY(kx_linear(f32, down, rows, st));
+    }
+    if (record) {
+      hipLaunchKernelGGL(sum_streams_k, dim3(T), dim3(256), 0, st, streams, record + ((size_t)i * max_context + pos) * max_batch * W, W, S, batch, max_batch);
+      KX_LAUNCH_CHECK();
+    }
+  }
+  hist_cur ^= 1;
+  x_row0 = (C - 1) * batch;
+  if (sample) {
+    KX_TRY(logits_of(streams + (size_t)x_row0 * S * W, nullptr, batch, logits));
+    KX_TRY(kx_argmax_launch(logits, batch, c.vocab, c.vocab, next, argmax_scratch, st));
+  }
+  sampled = sample;
+  pos += C;
+  return KX_OK;
+}
+
+int HybridModel::row_logits(const int *token_rows, int n, float *d_out) {
+  KX_HIP(hipMemcpyAsync(want, token_rows, (size_t)n * 4, hipMemcpyHostToDevice, st));
+  KX_HIP(hipStreamSynchronize(st));
+  return logits_of(streams, want, n, d_out);
+}
+
+int HybridModel::hidden_bf16(uint16_t *h_out) {
+  std::vector<float> x((size_t)batch * c.streams * c.width);
+  KX_HIP(hipMemcpyAsync(x.data(), streams + (size_t)x_row0 * c.streams * c.width, x.size() * 4, hipMemcpyDeviceToHost, st));
+  KX_HIP(hipStreamSynchronize(st));
+  for (int b = 0; b < batch; ++b)
+    for (int k = 0; k < c.width; ++k) {
+      float v = 0.0f;
+      for (int s = 0; s < c.streams; ++s) v += x[((size_t)b * c.streams + s) * c.width + k];
+      h_out[(size_t)b * c.width + k] = kx_bf16_rne(v);
+    }
+  return KX_OK;
+}
+
+int HybridModel::set_residual_record(bool on) {
+  KX_HIP(hipStreamSynchronize(st));
+  if (!on) {
+    if (record) KX_HIP(hipFree(record));
+    record = nullptr;
+  } else if (!record) {
+    const size_t bytes = (size_t)n_layers * max_context * max_batch * c.width * 4;
+    KX_HIP(hipMalloc((void **)&record, bytes));
+    KX_HIP(hipMemset(record, 0, bytes));
+  }
+  return KX_OK;
+}
+int HybridModel::residual(int layer, int pos0, int n, float *h_out) {
+  KX_REQUIRE(record, "kx_model_residual: the record is off (kx_model_set_residual_record)");
+  const size_t row = (size_t)c.width * 4;
+  KX_HIP(hipMemcpy2DAsync(h_out, batch * row, record + ((size_t)layer * max_context + pos0) * max_batch * c.width, max_batch * row, batch * row, n,
+                          hipMemcpyDeviceToHost, st));
+  KX_HIP(hipStreamSynchronize(st));
+  return KX_OK;
+}
+
+int hybrid_open(const char *name, const std::string &dir, const KxHybridConfig &config, const kx_open_options &o, kx_model **out) {
+  KX_REQUIRE((size_t)o.layers <= config.layers.size(), "kx_model_open: the model has %zu layers, %d asked for", config.layers.size(), o.layers);
+  HybridModel *m = new HybridModel();
+  m->name = name;
+  m->c = config;
+  if (o.layers) m->c.layers.resize(o.layers);
+  m->n_layers = (int)m->c.layers.size(); m->hidden = config.width; m->vocab = config.vocab;
+  m->max_batch = o.max_batch; m->max_context = o.max_context; m->eos_id = o.eos_id;
+  m->dtype = o.dtype; m->f32 = o.dtype == KX_DTYPE_F32;
+  m->step_tokens = (int)std::min<int64_t>(std::max(o.step_tokens, o.max_batch), (int64_t)o.max_context * o.max_batch);
+  m->prefill_chunk = m->step_tokens;
+  m->part_tokens = std::max(o.max_batch, std::min(64, m->step_tokens));
+  m->init_sigma_ = o.init_sigma;
+  auto build = [&]() -> int {
+    const size_t total = m->layout(nullptr);
+    size_t free_b = 0, total_b = 0;
+    KX_HIP(hipMemGetInfo(&free_b, &total_b));
+    KX_REQUIRE(total + ((size_t)1 << 30) <= free_b, "kx_model_open: the model needs %.1f GB of HBM, %.1f GB are free", total / 1e9, free_b / 1e9);
+    KX_HIP(hipMalloc((void **)&m->arena, total));
+    KX_TRY(kx_model_resources(m, "kx_model_open"));
+    KX_HIP(hipMemsetAsync(m->arena, 0, total, m->st));  // padding stays zero, cache rows that were never written are finite
+    m->layout(m->arena);
+    KX_TRY(m->fill(dir, o));
+    KX_HIP(hipStreamSynchronize(m->st));
+    return KX_OK;
+  };
+  const int rc = build();
+  if (rc) {
+    delete m;
+    return rc;
+  }
+  *out = m;
+  return KX_OK;
+}
+
+int kagalorn_open(const std::string &dir, const KxJson &json, const kx_open_options &o, kx_model **out) {
+  KxHybridConfig c;
+  KX_TRY(kx_kagalorn_config(json, c));
+  return hybrid_open("Kagalorn", dir, c, o, out);
+}
+
+const KxDesignEntry entry(KxDesign{"Kagalorn", kx_kagalorn_matches, kagalorn_open});
+
+}  // namespace

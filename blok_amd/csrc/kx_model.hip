@@ -1,4 +1,4 @@
-// kx_model.hip -- the decoder stack: prefill, decode step, greedy sample, generate.
+// kx_model.hip -- the Kimi-K2 design: weights, cache and one step of the stack (the loops around it: kx_stack.hip).
 //
 // Reference: generate() and its run() lambda, src/kimi_exec.cu:780-893.  The
 // reference allocates 19 single-token fp32 scratch buffers (:792-799), streams
@@ -28,6 +28,8 @@
 #include "kx_index.h"
 #include "kx_load.h"
 #include "kx_mla.h"
+#include "kx_argmax.h"
+#include "kx_model.h"
 
 namespace {
 
@@ -61,23 +63,18 @@ __global__ void head_groups_k(int tokens, int heads, int4 *__restrict__ work, in
   pairs[idx] = t * heads + h;
   if (t == 0) work[h] = make_int4(h, h * tokens, (h + 1) * tokens, h);
 }
-__global__ void copy_ids_k(const uint32_t *__restrict__ src, uint32_t *__restrict__ dst, int n) {
-  int i = blockIdx.x * blockDim.x + threadIdx.x;
-  if (i < n) dst[i] = src[i];
-}
 
 }  // namespace
 
-struct kx_model {
+namespace {
+
+struct KimiModel : kx_model {
   kx_config c;
-  char *arena = nullptr;
-  size_t arena_bytes = 0;
   uint16_t *embed, *final_norm, *lm_head, *rope_tab;
   std::vector<Layer> layers;
   // scratch of one step
   uint16_t *x, *n, *qkv, *qa, *q, *o_lat, *att, *dmid;
-  float *qabs, *partial, *logits, *argmax_scratch;
-  uint32_t *ids, *next, *history;  // [max_context][B], [B], [max_context][B]
+  float *qabs, *partial;
   int *head_count;                 // [heads] arrival counters of the q_b GEMV that finishes the query; zero between launches
   int *hand_err;                   // error flag of the resident launches (kx_front.hip, kx_i4.hip): a wait for another workgroup's values gave up
   uint32_t *front_hand;            // tagged words of the attention block's front launch (q_a, kv_a, q)
@@ -92,20 +89,27 @@ struct kx_model {
   int *route_distinct = nullptr;   // [n_layers] distinct experts of the last step
   float *route_history = nullptr;  // record level 2: router logits of every position, [n_layers][max_context][max_batch][experts]
   kx_moe_workspace *moe_ws = nullptr;
-  hipStream_t st = nullptr;
-  hipEvent_t ev[3] = {nullptr, nullptr, nullptr};
-  int batch = 0, pos = 0;
-  int prefill_chunk = 1;  // prompt positions per prefill step (kx_model_set_prefill_chunk)
   uint32_t exact = 0;     // kx_model_set_exact: KX_EXACT_* parts that keep the bit-reproducible kernels at every batch size
-  int x_row0 = 0;         // first row of x that belongs to the last position of the last step
-  bool sampled = false;
-  float ms_prefill = 0, ms_decode = 0;
-  int steps_decoded = 0;  // ids sampled per sequence by the last kx_generate (less than asked for when every sequence ended)
-  uint64_t load_bytes = 0;  // checkpoint bytes copied in by kx_model_load, and the time that took
-  double load_seconds = 0;
+
+  ~KimiModel() override;
+  const char *design() const override { return "Kimi-K2"; }
+  int step(const uint32_t *d_ids, bool sample, int C) override;
+  int step_positions(int batch_) const override;
+  int row_logits(const int *rows, int n_rows, float *d_out) override;
+  int device_error() override;
+  int rewind(int positions) override { return KX_OK; }  // rows above the current position are never read
+  int hidden_bf16(uint16_t *h_out) override;
 };
 
-namespace {
+// the Kimi model behind a handle, or nullptr with the message set
+KimiModel *kimi(kx_model *m, const char *who) {
+  KimiModel *k = m ? dynamic_cast<KimiModel *>(m) : nullptr;
+  if (!k) kx_set_error(m ? "%s: not available for this design" : "%s: null model", who);
+  return k;
+}
+#define KX_KIMI(var, handle, who) \
+  KimiModel *var = kimi(handle, who); \
+  if (!var) return KX_ERR_ARG
 
 // tokens a step may carry: a decode step has one per sequence, a prefill step up to this many (positions x sequences)
 constexpr int STEP_TOKENS = 2048;
@@ -114,13 +118,8 @@ inline int step_tokens(const kx_config *c) { return c->max_batch > STEP_TOKENS ?
 constexpr int ATT_ENTRIES = 256;
 inline int att_entries(const kx_config *c) { return c->max_batch > ATT_ENTRIES ? c->max_batch : ATT_ENTRIES; }
 
-struct Plan {  // byte offsets of everything in the arena
-  size_t total = 0, weights = 0, cache = 0, scratch = 0;
-  size_t take(size_t bytes) {
-    size_t at = total;
-    total += (bytes + 255) & ~(size_t)255;
-    return at;
-  }
+struct Plan : KxPlan {
+  size_t weights = 0, cache = 0, scratch = 0;
 };
 
 int check_model_cfg(const kx_config *c) {
@@ -143,7 +142,7 @@ int check_model_cfg(const kx_config *c) {
 }
 
 // lays the model out; when m != nullptr also sets its pointers (arena must be allocated)
-int layout(const kx_config *c, Plan &p, kx_model *m) {
+int layout(const kx_config *c, Plan &p, KimiModel *m) {
   const size_t H = c->hidden, V = c->vocab, E = c->experts, I = c->moe_inter, SI = c->shared_inter, D = c->dense_inter;
   const size_t KD = (size_t)c->heads * (c->qk_nope + c->qk_rope), VD = (size_t)c->heads * c->v_head;
   const size_t KVA = c->kv_rank + c->qk_rope, KVB = (size_t)c->heads * (c->qk_nope + c->v_head), B = c->max_batch;
@@ -223,7 +222,7 @@ int layout(const kx_config *c, Plan &p, kx_model *m) {
 }
 
 // rope table for every position, computed on the host
-int init_rope(kx_model *m) {
+int init_rope(KimiModel *m) {
   const kx_config &c = m->c;
   std::vector<uint16_t> tab((size_t)c.max_context * c.qk_rope);
   int rc = kx_rope_table(&c, 0, c.max_context, tab.data());
@@ -233,7 +232,7 @@ int init_rope(kx_model *m) {
   return KX_OK;
 }
 
-int init_weights(kx_model *m) {
+int init_weights(KimiModel *m) {
   const kx_config &c = m->c;
   const size_t H = c.hidden, V = c.vocab, E = c.experts, I = c.moe_inter, SI = c.shared_inter, D = c.dense_inter;
   const size_t KD = (size_t)c.heads * (c.qk_nope + c.qk_rope), VD = (size_t)c.heads * c.v_head;
@@ -285,7 +284,10 @@ int init_weights(kx_model *m) {
 // position pos + i of sequence b).  Everything but the attention is per token, so the step runs as a batch of B * C
 // tokens; the q absorb writes the cache rows of all C positions, then position i attends to rows 0 .. pos + i (one
 // launch each, the kernels take the position from the token index).  Only the last position is sampled.
-int step(kx_model *m, const uint32_t *d_ids, bool sample, int C = 1) {
+}  // namespace
+
+int KimiModel::step(const uint32_t *d_ids, bool sample, int C) {
+  KimiModel *const m = this;
   const kx_config &c = m->c;
   const int NB = m->batch, B = NB * C, H = c.hidden, pos = m->pos;
   const int KD = c.heads * (c.qk_nope + c.qk_rope), VD = c.heads * c.v_head, KVA = c.kv_rank + c.qk_rope;
@@ -463,7 +465,27 @@ int step(kx_model *m, const uint32_t *d_ids, bool sample, int C = 1) {
   return KX_OK;
 }
 
-}  // namespace
+int KimiModel::step_positions(int batch_) const {
+  return exact == KX_EXACT_ALL ? 1 : STEP_TOKENS / batch_;  // a step of several positions is a tolerance path
+}
+
+int KimiModel::row_logits(const int *rows, int n_rows, float *d_out) {
+  for (int i = 0; i < n_rows; ++i) {
+    KxGemvArgs g = {};
+    g.w0 = lm_head; g.x = x + (size_t)rows[i] * c.hidden; g.x_stride = c.hidden; g.out = d_out + (size_t)i * c.vocab; g.out_stride = c.vocab;
+    g.rows = c.vocab; g.cols = c.hidden; g.tokens = 1; g.norm_w = final_norm; g.norm_eps = c.rms_eps;
+    int rc = kx_gemv_launch(KX_EPI_ARGMAX, g, st);
+    if (rc) return rc;
+  }
+  return KX_OK;
+}
+
+KimiModel::~KimiModel() {
+  if (moe_ws) kx_moe_workspace_destroy(moe_ws);
+  if (route_logits) (void)hipFree(route_logits);
+  if (route_distinct) (void)hipFree(route_distinct);
+  if (route_history) (void)hipFree(route_history);
+}
 
 extern "C" int kx_model_bytes(const kx_config *cfg, uint64_t *weights, uint64_t *kv_cache, uint64_t *scratch) {
   int rc = check_model_cfg(cfg);
@@ -477,7 +499,7 @@ extern "C" int kx_model_bytes(const kx_config *cfg, uint64_t *weights, uint64_t 
 }
 
 // allocates the arena, lays the model out and creates its stream, events and MoE workspace; weights are not set
-static int model_new(const kx_config *cfg, const char *who, kx_model **out) {
+static int model_new(const kx_config *cfg, const char *who, KimiModel **out) {
   KX_REQUIRE(out, "%s: null out pointer", who);
   *out = nullptr;
   int rc = check_model_cfg(cfg);
@@ -488,21 +510,20 @@ static int model_new(const kx_config *cfg, const char *who, kx_model **out) {
   KX_HIP(hipMemGetInfo(&free_b, &total_b));
   KX_REQUIRE(p.total + ((size_t)1 << 30) <= free_b, "%s: the model needs %.1f GB of HBM, %.1f GB are free", who,
              p.total / 1e9, free_b / 1e9);
-  kx_model *m = new kx_model();
+  KimiModel *m = new KimiModel();
   m->c = *cfg;
+  m->n_layers = cfg->n_layers; m->hidden = cfg->hidden; m->vocab = cfg->vocab; m->max_batch = cfg->max_batch;
+  m->max_context = cfg->max_context; m->eos_id = cfg->eos_id; m->step_tokens = STEP_TOKENS;
+  m->weight_bytes = p.weights; m->cache_bytes = p.cache; m->scratch_bytes = p.scratch;
   hipError_t e = hipMalloc((void **)&m->arena, p.total);
   if (e != hipSuccess) {
     kx_set_error("%s: hipMalloc(%zu): %s", who, p.total, hipGetErrorString(e));
     delete m;
     return KX_ERR_HIP;
   }
-  m->arena_bytes = p.total;
   Plan p2;
   layout(cfg, p2, m);
-  rc = KX_OK;
-  if (hipStreamCreate(&m->st) != hipSuccess) rc = KX_ERR_HIP;
-  for (auto &ev : m->ev)
-    if (!rc && hipEventCreate(&ev) != hipSuccess) rc = KX_ERR_HIP;
+  rc = kx_model_resources(m, who);
   if (!rc && cfg->first_dense < cfg->n_layers) rc = kx_moe_workspace_create(cfg, step_tokens(cfg), &m->moe_ws);
   if (!rc && m->moe_ws) kx_moe_workspace_set_err(m->moe_ws, m->hand_err);
   if (!rc && (hipMemsetAsync(m->head_count, 0, (size_t)cfg->heads * 4, m->st) != hipSuccess ||
@@ -520,7 +541,7 @@ static int model_new(const kx_config *cfg, const char *who, kx_model **out) {
 }
 
 extern "C" int kx_model_create(const kx_config *cfg, kx_model **out) {
-  kx_model *m = nullptr;
+  KimiModel *m = nullptr;
   int rc = model_new(cfg, "kx_model_create", &m);
   if (rc) return rc;
   if ((rc = init_weights(m))) {
@@ -532,7 +553,7 @@ extern "C" int kx_model_create(const kx_config *cfg, kx_model **out) {
 }
 
 // where checkpoint tensor `n` lives in the arena
-static char *need_dst(kx_model *m, const KxNeed &n) {
+static char *need_dst(KimiModel *m, const KxNeed &n) {
   const kx_config &c = m->c;
   const size_t H = c.hidden, I = c.moe_inter, e = n.expert < 0 ? 0 : (size_t)n.expert;
   if (n.layer < 0) return (char *)(n.slot == KXS_EMBED ? m->embed : n.slot == KXS_FINAL_NORM ? m->final_norm : m->lm_head);
@@ -575,7 +596,7 @@ extern "C" int kx_model_load(const kx_config *cfg, const char *index_path, kx_mo
   if (rc) return rc;
   std::vector<KxNeed> needs;
   if ((rc = check_model_cfg(cfg)) || (rc = kx_index_contract(ix, cfg, needs))) return rc;
-  kx_model *m = nullptr;
+  KimiModel *m = nullptr;
   if ((rc = model_new(cfg, "kx_model_load", &m))) return rc;
   std::vector<KxLoadItem> items;
   items.reserve(needs.size());
@@ -596,40 +617,12 @@ extern "C" int kx_model_load(const kx_config *cfg, const char *index_path, kx_mo
   return KX_OK;
 }
 
-extern "C" int kx_model_load_info(kx_model *m, uint64_t *bytes, double *seconds) {
-  KX_REQUIRE(m, "kx_model_load_info: null model");
-  if (bytes) *bytes = m->load_bytes;
-  if (seconds) *seconds = m->load_seconds;
-  return KX_OK;
-}
-
-extern "C" int kx_model_destroy(kx_model *m) {
-  if (!m) return KX_OK;
-  if (m->st) (void)hipStreamSynchronize(m->st);
-  if (m->moe_ws) kx_moe_workspace_destroy(m->moe_ws);
-  for (auto &ev : m->ev)
-    if (ev) (void)hipEventDestroy(ev);
-  if (m->st) (void)hipStreamDestroy(m->st);
-  if (m->arena) (void)hipFree(m->arena);
-  if (m->route_logits) (void)hipFree(m->route_logits);
-  if (m->route_distinct) (void)hipFree(m->route_distinct);
-  if (m->route_history) (void)hipFree(m->route_history);
-  delete m;
-  return KX_OK;
-}
-
-static int check_ids(const kx_model *m, const uint32_t *ids, size_t n) {
-  for (size_t i = 0; i < n; ++i)
-    KX_REQUIRE(ids[i] < (uint32_t)m->c.vocab, "token id %u outside the vocabulary of %d", ids[i], m->c.vocab);  // :552, :652
-  return KX_OK;
-}
-
-// Synchronises the model's stream and reports a wait inside a resident launch (kx_front.hip, the routed experts'
-// launch of kx_i4.hip) that was given up: the steps since then computed with values that were not there yet.
-static int check_front(kx_model *m) {
+// Reports a wait inside a resident launch (kx_front.hip, the routed experts' launch of kx_i4.hip) that was given up:
+// the steps since then computed with values that were not there yet.
+int KimiModel::device_error() {
   int flag = 0;
-  KX_HIP(hipMemcpyAsync(&flag, m->hand_err, 4, hipMemcpyDeviceToHost, m->st));
-  KX_HIP(hipStreamSynchronize(m->st));
+  KX_HIP(hipMemcpyAsync(&flag, hand_err, 4, hipMemcpyDeviceToHost, st));
+  KX_HIP(hipStreamSynchronize(st));
   if (flag) {
     kx_set_error("kx_model: a workgroup of a resident launch gave up waiting for values from the others (not all workgroups of the launch "
                  "were on the device at once); results since then are invalid -- switch the resident launches off with "
@@ -639,155 +632,30 @@ static int check_front(kx_model *m) {
   return KX_OK;
 }
 
-extern "C" int kx_prefill(kx_model *m, const uint32_t *h_ids, int32_t batch, int32_t prompt_len) {
-  KX_REQUIRE(m && h_ids, "kx_prefill: null argument");
-  KX_REQUIRE(batch > 0 && batch <= m->c.max_batch, "kx_prefill: batch=%d outside [1, %d]", batch, m->c.max_batch);
-  KX_REQUIRE(prompt_len > 0 && prompt_len <= m->c.max_context, "kx_prefill: prompt_len=%d outside [1, %d]", prompt_len, m->c.max_context);  // :555, :784
-  int rc = check_ids(m, h_ids, (size_t)batch * prompt_len);
-  if (rc) return rc;
-  std::vector<uint32_t> pm((size_t)prompt_len * batch);  // position-major
-  for (int b = 0; b < batch; ++b)
-    for (int i = 0; i < prompt_len; ++i) pm[(size_t)i * batch + b] = h_ids[(size_t)b * prompt_len + i];
-  KX_HIP(hipMemcpyAsync(m->ids, pm.data(), pm.size() * 4, hipMemcpyHostToDevice, m->st));
-  KX_HIP(hipStreamSynchronize(m->st));  // pm goes out of scope
-  m->batch = batch;
-  m->pos = 0;
-  // :886: one run() per prompt token, sampling on the last; with a prefill chunk set, up to that many positions per step
-  int chunk = m->prefill_chunk < STEP_TOKENS / batch ? m->prefill_chunk : STEP_TOKENS / batch;
-  if (chunk < 1 || m->exact == KX_EXACT_ALL) chunk = 1;  // a step of several positions is a tolerance path
-  for (int i = 0; i < prompt_len; i += chunk) {
-    const int n = prompt_len - i < chunk ? prompt_len - i : chunk;
-    if ((rc = step(m, m->ids + (size_t)i * batch, i + n == prompt_len, n))) return rc;
-  }
-  return KX_OK;
-}
-
-extern "C" int kx_decode_step(kx_model *m, const uint32_t *h_ids) {
-  KX_REQUIRE(m, "kx_decode_step: null model");
-  KX_REQUIRE(m->batch > 0, "kx_decode_step: no prefill has run");
-  KX_REQUIRE(m->pos < m->c.max_context, "kx_decode_step: the context of %d positions is full", m->c.max_context);  // :784
-  const uint32_t *src = m->next;
-  if (h_ids) {
-    int rc = check_ids(m, h_ids, m->batch);
-    if (rc) return rc;
-    uint32_t *slot = m->ids + (size_t)m->pos * m->batch;
-    KX_HIP(hipMemcpyAsync(slot, h_ids, (size_t)m->batch * 4, hipMemcpyHostToDevice, m->st));
-    KX_HIP(hipStreamSynchronize(m->st));
-    src = slot;
-  } else {
-    KX_REQUIRE(m->sampled, "kx_decode_step: no sampled ids to feed (pass h_ids)");
-    // the sampler overwrites `next`; feed a copy
-    uint32_t *slot = m->ids + (size_t)m->pos * m->batch;
-    hipLaunchKernelGGL(copy_ids_k, dim3(kx_cdiv(m->batch, 64)), dim3(64), 0, m->st, m->next, slot, m->batch);
-    KX_LAUNCH_CHECK();
-    src = slot;
-  }
-  return step(m, src, true);
-}
-
-extern "C" int kx_greedy_sample(kx_model *m, uint32_t *h_out) {
-  KX_REQUIRE(m && h_out, "kx_greedy_sample: null argument");
-  KX_REQUIRE(m->sampled, "kx_greedy_sample: the last step did not sample");
-  KX_HIP(hipMemcpyAsync(h_out, m->next, (size_t)m->batch * 4, hipMemcpyDeviceToHost, m->st));
-  return check_front(m);
-}
-
-extern "C" int kx_generate(kx_model *m, const uint32_t *h_prompt, int32_t batch, int32_t prompt_len, int32_t n_tokens,
-                           int ignore_eos, uint32_t *h_out, int32_t *h_counts) {
-  KX_REQUIRE(m && h_prompt && h_out && h_counts, "kx_generate: null argument");
-  KX_REQUIRE(n_tokens > 0, "kx_generate: n_tokens=%d must be positive", n_tokens);  // :542
-  KX_REQUIRE((int64_t)prompt_len + n_tokens <= m->c.max_context, "requested sequence exceeds the context of %d positions", m->c.max_context);  // :784
-  int rc;
-  KX_HIP(hipEventRecord(m->ev[0], m->st));
-  if ((rc = kx_prefill(m, h_prompt, batch, prompt_len))) return rc;
-  KX_HIP(hipEventRecord(m->ev[1], m->st));
-  const int cp = kx_cdiv(batch, 64);
-  // Steps are enqueued without waiting for the host.  When the end-of-sequence id counts, the ids sampled so far are
-  // read back every eighth step, and the loop ends once every sequence has sampled it (:887-888 stop there too):
-  // at most eight steps are decoded for nothing.
-  std::vector<uint32_t> hist((size_t)n_tokens * batch);
-  std::vector<char> ended(batch, 0);
-  int made = 0, seen = 0;  // history rows written on the device, and of those, rows the host has read
-  auto read_back = [&]() -> int {
-    if (seen == made) return KX_OK;
-    KX_HIP(hipMemcpyAsync(hist.data() + (size_t)seen * batch, m->history + (size_t)seen * batch, (size_t)(made - seen) * batch * 4,
-                          hipMemcpyDeviceToHost, m->st));
-    KX_HIP(hipStreamSynchronize(m->st));
-    for (; seen < made; ++seen)
-      for (int b = 0; b < batch; ++b)
-        if (hist[(size_t)seen * batch + b] == m->c.eos_id) ended[b] = 1;
-    return KX_OK;
-  };
-  for (int i = 0; i < n_tokens; ++i) {  // :887-890
-    hipLaunchKernelGGL(copy_ids_k, dim3(cp), dim3(64), 0, m->st, m->next, m->history + (size_t)i * batch, batch);
-    KX_LAUNCH_CHECK();
-    made = i + 1;
-    if (!ignore_eos && (i & 7) == 7) {
-      if ((rc = read_back())) return rc;
-      bool all = true;
-      for (int b = 0; b < batch; ++b) all = all && ended[b];
-      if (all) break;
-    }
-    if (i + 1 < n_tokens && (rc = step(m, m->history + (size_t)i * batch, true))) return rc;
-  }
-  KX_HIP(hipEventRecord(m->ev[2], m->st));
-  if ((rc = read_back())) return rc;
-  if ((rc = check_front(m))) return rc;
-  KX_HIP(hipEventElapsedTime(&m->ms_prefill, m->ev[0], m->ev[1]));
-  KX_HIP(hipEventElapsedTime(&m->ms_decode, m->ev[1], m->ev[2]));
-  m->steps_decoded = made;
-  for (int b = 0; b < batch; ++b) {  // generation stops before the end-of-sequence id is emitted (:887-888)
-    int n = 0;
-    for (int i = 0; i < made; ++i) {
-      const uint32_t id = hist[(size_t)i * batch + b];
-      if (!ignore_eos && id == m->c.eos_id) break;
-      h_out[(size_t)b * n_tokens + n++] = id;
-    }
-    h_counts[b] = n;
-  }
-  return KX_OK;
-}
-
-extern "C" int kx_model_set_prefill_chunk(kx_model *m, int32_t positions) {
-  KX_REQUIRE(m, "kx_model_set_prefill_chunk: null model");
-  KX_REQUIRE(positions >= 1 && positions <= STEP_TOKENS, "kx_model_set_prefill_chunk: positions=%d outside [1, %d]", positions, STEP_TOKENS);
-  m->prefill_chunk = positions;
-  return KX_OK;
-}
-
-extern "C" int kx_model_set_exact(kx_model *m, uint32_t mask) {
-  KX_REQUIRE(m, "kx_model_set_exact: null model");
+extern "C" int kx_model_set_exact(kx_model *handle, uint32_t mask) {
+  KX_KIMI(m, handle, "kx_model_set_exact");
   KX_REQUIRE(!(mask & ~(uint32_t)KX_EXACT_ALL), "kx_model_set_exact: unknown bits in mask 0x%x", mask);
   m->exact = mask;
   return KX_OK;
 }
 
-extern "C" int kx_model_rewind(kx_model *m, int32_t positions) {
-  KX_REQUIRE(m, "kx_model_rewind: null model");
-  KX_REQUIRE(m->batch > 0, "kx_model_rewind: no prefill has run");
-  KX_REQUIRE(positions >= 0 && positions <= m->pos, "kx_model_rewind: positions=%d outside [0, %d]", positions, m->pos);
-  m->pos -= positions;
-  if (positions) m->sampled = false;  // the sampled ids belonged to the last position
-  return KX_OK;
-}
-
-extern "C" int kx_model_debug_fail_waits(kx_model *m) {
-  KX_REQUIRE(m, "kx_model_debug_fail_waits: null model");
+extern "C" int kx_model_debug_fail_waits(kx_model *handle) {
+  KX_KIMI(m, handle, "kx_model_debug_fail_waits");
   const int one = 1;
   KX_HIP(hipMemcpyAsync(m->hand_err, &one, 4, hipMemcpyHostToDevice, m->st));
   KX_HIP(hipStreamSynchronize(m->st));
   return KX_OK;
 }
 
-extern "C" int kx_model_set_attention_kernel(kx_model *m, int32_t kernel) {
-  KX_REQUIRE(m, "kx_model_set_attention_kernel: null model");
+extern "C" int kx_model_set_attention_kernel(kx_model *handle, int32_t kernel) {
+  KX_KIMI(m, handle, "kx_model_set_attention_kernel");
   KX_REQUIRE(kernel >= KX_MLA_AUTO && kernel <= KX_MLA_MATRIX_CORES, "kx_model_set_attention_kernel: kernel=%d outside [0, 2]", kernel);
   KX_REQUIRE(kernel != KX_MLA_MATRIX_CORES || m->c.heads == 64, "kx_model_set_attention_kernel: the matrix-core kernel is built for 64 heads (model: %d)", m->c.heads);
   m->mla_kernel = kernel;
   return KX_OK;
 }
-extern "C" int kx_model_set_routing_record(kx_model *m, int on) {
-  KX_REQUIRE(m, "kx_model_set_routing_record: null model");
+extern "C" int kx_model_set_routing_record(kx_model *handle, int on) {
+  KX_KIMI(m, handle, "kx_model_set_routing_record");
   KX_REQUIRE(m->c.first_dense < m->c.n_layers, "kx_model_set_routing_record: the model has no MoE layer");
   KX_HIP(hipStreamSynchronize(m->st));
   KX_REQUIRE(on >= 0 && on <= 2, "kx_model_set_routing_record: level %d outside [0, 2]", on);
@@ -821,7 +689,8 @@ extern "C" int kx_model_set_routing_record(kx_model *m, int on) {
   m->route_logits = lg; m->route_distinct = di;
   return KX_OK;
 }
-extern "C" int kx_model_routing(kx_model *m, int32_t layer, float *h_logits, int32_t *h_distinct) {
+extern "C" int kx_model_routing(kx_model *handle, int32_t layer, float *h_logits, int32_t *h_distinct) {
+  KX_KIMI(m, handle, "kx_model_routing");
   KX_REQUIRE(m && m->route_logits, "kx_model_routing: null model, or kx_model_set_routing_record was not switched on");
   KX_REQUIRE(layer >= m->c.first_dense && layer < m->c.n_layers, "kx_model_routing: layer %d is not a MoE layer of this model", layer);
   KX_REQUIRE(m->batch > 0, "kx_model_routing: no step has run");
@@ -832,7 +701,8 @@ extern "C" int kx_model_routing(kx_model *m, int32_t layer, float *h_logits, int
   KX_HIP(hipStreamSynchronize(m->st));
   return KX_OK;
 }
-extern "C" int kx_model_routing_history(kx_model *m, int32_t layer, int32_t pos0, int32_t n, float *h_logits) {
+extern "C" int kx_model_routing_history(kx_model *handle, int32_t layer, int32_t pos0, int32_t n, float *h_logits) {
+  KX_KIMI(m, handle, "kx_model_routing_history");
   KX_REQUIRE(m && h_logits && m->route_history, "kx_model_routing_history: null argument, or kx_model_set_routing_record is not at level 2");
   KX_REQUIRE(layer >= m->c.first_dense && layer < m->c.n_layers, "kx_model_routing_history: layer %d is not a MoE layer of this model", layer);
   KX_REQUIRE(pos0 >= 0 && n >= 0 && pos0 + n <= m->c.max_context, "kx_model_routing_history: positions [%d, %d) outside the context of %d", pos0, pos0 + n, m->c.max_context);
@@ -841,39 +711,20 @@ extern "C" int kx_model_routing_history(kx_model *m, int32_t layer, int32_t pos0
   KX_HIP(hipStreamSynchronize(m->st));
   return KX_OK;
 }
-extern "C" int kx_model_set_fusion(kx_model *m, uint32_t mask) {
-  KX_REQUIRE(m, "kx_model_set_fusion: null model");
+extern "C" int kx_model_set_fusion(kx_model *handle, uint32_t mask) {
+  KX_KIMI(m, handle, "kx_model_set_fusion");
   KX_REQUIRE(!(mask & ~(uint32_t)KX_FUSE_ALL), "kx_model_set_fusion: unknown bits in mask 0x%x", mask);
   m->fusion = mask;
   return KX_OK;
 }
 
-extern "C" int kx_model_steps_decoded(kx_model *m, int32_t *steps) {
-  KX_REQUIRE(m && steps, "kx_model_steps_decoded: null argument");
-  *steps = m->steps_decoded;
+int KimiModel::hidden_bf16(uint16_t *h_out) {
+  KX_HIP(hipMemcpyAsync(h_out, x + (size_t)x_row0 * c.hidden, (size_t)batch * c.hidden * 2, hipMemcpyDeviceToHost, st));
+  KX_HIP(hipStreamSynchronize(st));
   return KX_OK;
 }
-
-extern "C" int kx_model_timing(kx_model *m, float *ms2) {
-  KX_REQUIRE(m && ms2, "kx_model_timing: null argument");
-  ms2[0] = m->ms_prefill;
-  ms2[1] = m->ms_decode;
-  return KX_OK;
-}
-
-extern "C" int kx_model_hidden(kx_model *m, uint16_t *h_out) {
-  KX_REQUIRE(m && h_out && m->batch > 0, "kx_model_hidden: null argument or no step has run");
-  KX_HIP(hipMemcpyAsync(h_out, m->x + (size_t)m->x_row0 * m->c.hidden, (size_t)m->batch * m->c.hidden * 2, hipMemcpyDeviceToHost, m->st));
-  KX_HIP(hipStreamSynchronize(m->st));
-  return KX_OK;
-}
-extern "C" int kx_model_logits(kx_model *m, float *h_out) {
-  KX_REQUIRE(m && h_out && m->sampled, "kx_model_logits: null argument or the last step did not sample");
-  KX_HIP(hipMemcpyAsync(h_out, m->logits, (size_t)m->batch * m->c.vocab * 4, hipMemcpyDeviceToHost, m->st));
-  KX_HIP(hipStreamSynchronize(m->st));
-  return KX_OK;
-}
-extern "C" int kx_model_latent(kx_model *m, int32_t layer, int32_t seq_index, int32_t pos0, int32_t n, uint16_t *h_out) {
+extern "C" int kx_model_latent(kx_model *handle, int32_t layer, int32_t seq_index, int32_t pos0, int32_t n, uint16_t *h_out) {
+  KX_KIMI(m, handle, "kx_model_latent");
   KX_REQUIRE(m && h_out, "kx_model_latent: null argument");
   KX_REQUIRE(layer >= 0 && layer < m->c.n_layers && seq_index >= 0 && seq_index < m->c.max_batch && pos0 >= 0 && n >= 0 &&
                  pos0 + n <= m->c.max_context, "kx_model_latent: index out of range");
@@ -883,8 +734,30 @@ extern "C" int kx_model_latent(kx_model *m, int32_t layer, int32_t seq_index, in
   KX_HIP(hipStreamSynchronize(m->st));
   return KX_OK;
 }
-extern "C" int kx_model_stream(kx_model *m, void **stream) {
-  KX_REQUIRE(m && stream, "kx_model_stream: null argument");
-  *stream = (void *)m->st;
-  return KX_OK;
+
+// ---- registry: a checkpoint directory (config.json of Kimi-K2, runtime-index.blok beside it) ----
+namespace {
+
+bool kimi_matches(const KxJson &config) {
+  const KxJson *t = config.get("text_config");
+  const KxJson *mt = (t ? *t : config).get("model_type");
+  return mt && mt->is(KxJson::STRING) && mt->str == "kimi_k2";
 }
+
+int kimi_open(const std::string &dir, const KxJson &config, const kx_open_options &o, kx_model **out) {
+  KX_REQUIRE(o.dtype == KX_DTYPE_BF16, "kx_model_open: Kimi-K2 runs in bfloat16 only");
+  KX_REQUIRE(!o.random_init, "kx_model_open: a random-init Kimi-K2 is made by kx_model_create");
+  const std::string index = dir + "/runtime-index.blok";
+  kx_config c;
+  int rc = kx_config_default(&c);
+  if (rc || (rc = kx_index_infer_config(index.c_str(), &c))) return rc;
+  KX_REQUIRE(o.layers <= c.n_layers, "kx_model_open: the checkpoint has %d layers, %d asked for", c.n_layers, o.layers);
+  if (o.layers) c.n_layers = o.layers;
+  c.max_batch = o.max_batch;
+  c.max_context = o.max_context;
+  return kx_model_load(&c, index.c_str(), out);
+}
+
+const KxDesignEntry entry(KxDesign{"Kimi-K2", kimi_matches, kimi_open});
+
+}  // namespace

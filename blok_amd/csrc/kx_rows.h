@@ -1,0 +1,129 @@
+// kx_rows.h -- activation rows of the hybrid decoder, built by one workgroup: what a matrix product reads as its
+// input.  The same code fills a row in LDS (the prologue of a decode GEMV, kx_linear.hip) and in memory (row_k, for
+// steps of many tokens).  No counterpart in the reference, whose decoder has one residual stream.
+//
+//   NORM   h = w * groupnorm(sum_s in[s] x_s): the input of a sublayer with several residual streams
+//   GATED  per head: the delta rule's read-out over its root mean square, times a weight, times silu(gate)
+//   PLAIN  a row that is in memory already
+// Rows are padded to the matrix's leading dimension; pad columns are zero (or, in memory, finite: the matrix's pad
+// columns are zero).
+#pragma once
+#include "kx_linear.h"
+#include "kx_math.h"
+#include "kx_wave.h"
+
+namespace kxr {
+
+typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
+
+template <class T> struct Elem;
+template <> struct Elem<uint16_t> {
+  static __device__ __forceinline__ float load(const uint16_t *p) { return kx_bf16_f32(*p); }
+  static __device__ __forceinline__ uint16_t make(float v) { return kx_bf16_rne(v); }
+  // eight elements of a weight stream, as they come
+  struct Raw { u32x4 a; };
+  static __device__ __forceinline__ Raw zero() { return Raw{u32x4{0, 0, 0, 0}}; }
+  static __device__ __forceinline__ Raw stream(const uint16_t *p) { return Raw{__builtin_nontemporal_load((const u32x4 *)p)}; }
+  static __device__ __forceinline__ Raw cached(const uint16_t *p) { return Raw{*(const u32x4 *)p}; }
+  static __device__ __forceinline__ void unpack(float (&f)[8], const Raw &r) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      f[2 * i] = kx_bits_f32(r.a[i] << 16);
+      f[2 * i + 1] = kx_bits_f32(r.a[i] & 0xffff0000u);
+    }
+  }
+};
+template <> struct Elem<float> {
+  static __device__ __forceinline__ float load(const float *p) { return *p; }
+  static __device__ __forceinline__ float make(float v) { return v; }
+  struct Raw { u32x4 a, b; };
+  static __device__ __forceinline__ Raw zero() { return Raw{u32x4{0, 0, 0, 0}, u32x4{0, 0, 0, 0}}; }
+  static __device__ __forceinline__ Raw stream(const float *p) {
+    return Raw{__builtin_nontemporal_load((const u32x4 *)p), __builtin_nontemporal_load((const u32x4 *)(p + 4))};
+  }
+  static __device__ __forceinline__ Raw cached(const float *p) { return Raw{((const u32x4 *)p)[0], ((const u32x4 *)p)[1]}; }
+  static __device__ __forceinline__ void unpack(float (&f)[8], const Raw &r) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      f[i] = kx_bits_f32(r.a[i]);
+      f[4 + i] = kx_bits_f32(r.b[i]);
+    }
+  }
+};
+
+// sum over the lanes of a wave, in every lane
+__device__ __forceinline__ float wave_sum(float v) {
+  float t = v;
+  kxw::swap_halves32(v, t);
+  v += t;
+  t = v;
+  kxw::swap_rows16(v, t);
+  v += t;
+  v += kxw::dpp_f<kxw::DPP_ROW_MIRROR>(v);
+  v += kxw::dpp_f<kxw::DPP_ROW_HALF_MIRROR>(v);
+  v += kxw::dpp_f<kxw::DPP_QUAD_XOR2>(v);
+  v += kxw::dpp_f<kxw::DPP_QUAD_XOR1>(v);
+  return v;
+}
+// sum over a workgroup, in every thread; red: one float per wave
+__device__ __forceinline__ float block_sum(float v, float *red) {
+  v = wave_sum(v);
+  const int nw = blockDim.x >> 6;
+  __syncthreads();  // red may still be read from the last call
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  float s = red[0];
+  for (int w = 1; w < nw; ++w) s += red[w];
+  return s;
+}
+
+// Row `tok` into dst[0 .. ld).  u: LDS scratch of kx_row_scratch(a) floats.  Whole workgroup; ends with a barrier.
+template <class T>
+__device__ __forceinline__ void build_row(const KxRowArgs &a, int tok, T *dst, int ld, float *u) {
+  const int tid = threadIdx.x, n = blockDim.x, lane = tid & 63, wave = tid >> 6, nw = n >> 6;
+  if (a.rows_map) tok = a.rows_map[tok];
+  if (a.kind == KX_ROW_NORM) {
+    float *part = u + a.cols;
+    const float *x = a.streams + (size_t)tok * a.n_streams * a.cols;
+    const int gs = a.cols / a.groups, spg = max(1, nw / a.groups), units = a.groups * spg, per = (gs + spg - 1) / spg;
+    for (int k = wave; k < units; k += nw) {  // a wave takes a slice of one group
+      const int g = k / spg, s = k - g * spg, hi = min(gs, (s + 1) * per);
+      float v = 0.0f;
+      for (int j = s * per + lane; j < hi; j += 64) {
+        const int c = g * gs + j;
+        float y = 0.0f;
+        for (int t = 0; t < a.n_streams; ++t) y = __builtin_fmaf(a.in ? a.in[t] : 1.0f, x[(size_t)t * a.cols + c], y);
+        u[c] = y;
+        v = __builtin_fmaf(y, y, v);
+      }
+      v = wave_sum(v);
+      if (lane == 0) part[k] = v;
+    }
+    __syncthreads();
+    for (int g = tid; g < a.groups; g += n) {
+      float s = part[g * spg];
+      for (int j = 1; j < spg; ++j) s += part[g * spg + j];
+      part[g * spg] = kx_rsqrtf(s / (float)gs + a.eps);
+    }
+    __syncthreads();
+    for (int c = tid; c < ld; c += n) dst[c] = Elem<T>::make(c < a.cols ? u[c] * part[(c / gs) * spg] * a.w[c] : 0.0f);
+  } else if (a.kind == KX_ROW_GATED) {
+    const float *o = a.o + (size_t)tok * a.cols, *gate = a.gate + (size_t)tok * a.gate_ld;
+    for (int h = wave; h < a.heads; h += nw) {
+      float v = 0.0f;
+      for (int d = lane; d < a.vdim; d += 64) v = __builtin_fmaf(o[h * a.vdim + d], o[h * a.vdim + d], v);
+      const float sc = kx_rsqrtf(wave_sum(v) / (float)a.vdim + a.eps);
+      for (int d = lane; d < a.vdim; d += 64) {
+        const int c = h * a.vdim + d;
+        dst[c] = Elem<T>::make(o[c] * sc * a.w[d] * kx_siluf(gate[c]));
+      }
+    }
+    for (int c = a.cols + tid; c < ld; c += n) dst[c] = Elem<T>::make(0.0f);
+  } else {
+    const T *x = (const T *)a.x + (size_t)tok * a.x_ld;
+    for (int c = tid * 8; c < ld; c += n * 8) *(typename Elem<T>::Raw *)(dst + c) = Elem<T>::cached(x + c);
+  }
+  __syncthreads();
+}
+
+}  // namespace kxr

@@ -38,6 +38,20 @@ class KxMoeWeights(C.Structure):
         "d_shared_down")]
 
 
+class KxOpenOptions(C.Structure):
+    _fields_ = [("dtype", C.c_int32), ("max_batch", C.c_int32), ("max_context", C.c_int32), ("step_tokens", C.c_int32),
+                ("layers", C.c_int32), ("eos_id", C.c_uint32), ("random_init", C.c_int32), ("init_sigma", C.c_float),
+                ("seed", C.c_uint64)]
+
+
+class KxModelShape(C.Structure):
+    _fields_ = [("design", C.c_char * 32)] + [(n, C.c_int32) for n in (
+        "n_layers", "hidden", "vocab", "dtype", "max_batch", "max_context", "step_tokens")] + [
+            (n, C.c_uint64) for n in ("weight_bytes", "cache_bytes", "scratch_bytes")]
+
+
+DTYPES = {"bfloat16": 0, "float32": 1}
+
 _P, _I, _U64, _F, _SZ = C.c_void_p, C.c_int32, C.c_uint64, C.c_float, C.c_size_t
 _PP = C.POINTER(C.c_void_p)
 _SIGS = {
@@ -105,6 +119,13 @@ _SIGS = {
     "kx_moe_decode_layer_timed": [C.POINTER(KxConfig), C.POINTER(KxMoeWeights), _P, _P, _P, _I,
                                   C.c_uint32, _P, C.POINTER(C.c_float)],
     "kx_moe_routed_only": [C.POINTER(KxConfig), C.POINTER(KxMoeWeights), _P, _P, _I, _I, _P],
+    "kx_open_options_default": [C.POINTER(KxOpenOptions)],
+    "kx_model_open": [C.c_char_p, C.POINTER(KxOpenOptions), _PP],
+    "kx_model_info": [_P, C.POINTER(KxModelShape)],
+    "kx_restart": [_P, _I],
+    "kx_extend": [_P, _P, _I, _P, _I, _P],
+    "kx_model_set_residual_record": [_P, C.c_int],
+    "kx_model_residual": [_P, _I, _I, _I, _P],
     "kx_index_check": [C.POINTER(KxConfig), C.c_char_p, C.POINTER(C.c_uint64), C.POINTER(C.c_uint64)],
     "kx_index_infer_config": [C.c_char_p, C.POINTER(KxConfig)],
     "kx_model_load": [C.POINTER(KxConfig), C.c_char_p, _PP],

@@ -266,6 +266,47 @@ int kx_decode_step(kx_model *model, const uint32_t *h_ids);
 int kx_greedy_sample(kx_model *model, uint32_t *h_out);
 int kx_generate(kx_model *model, const uint32_t *h_prompt, int32_t batch, int32_t prompt_len,
                 int32_t n_tokens, int ignore_eos, uint32_t *h_out, int32_t *h_counts);
+/* ---- model directories ---------------------------------------------------------------------
+ * kx_model_open  : reads <dir>/config.json, finds the design it names in the library's registry and opens the model
+ *                  with it.  Two designs are known: Kimi-K2 (config.json of the checkpoint with runtime-index.blok
+ *                  beside it; bfloat16) and Kagalorn (config.json and safetensors files; bfloat16 or float32).
+ *                  Every kx_model entry point works on the result; those that set up a mechanism only Kimi-K2 has
+ *                  (kx_model_set_fusion, _set_exact, _set_attention_kernel, routing, latent cache rows) return an error
+ *                  on another design.
+ * kx_model_info  : the opened model's shape.
+ * kx_restart     : forgets the sequences; the next kx_extend starts `batch` new ones at position 0.
+ * kx_extend      : appends n positions to every sequence; h_ids u32 [batch][n].  The positions are run in steps of up
+ *                  to the prefill chunk; where the cuts fall changes results by rounding only.  The last position
+ *                  is sampled.  h_want (n_want places among the n, the same for every sequence) asks for the logits at
+ *                  those places: h_logits f32 [n_want][batch][vocab]; the call synchronises when n_want > 0.       */
+#define KX_DTYPE_BF16 0 /* bf16 weights and activations, 32-bit accumulation, residual and state */
+#define KX_DTYPE_F32 1  /* everything in 32-bit */
+typedef struct kx_open_options {
+  int32_t dtype;       /* KX_DTYPE_*                                            */
+  int32_t max_batch;   /* sequences stepped together (1)                        */
+  int32_t max_context; /* positions per sequence (4096)                         */
+  int32_t step_tokens; /* most tokens a step carries; sizes the scratch (2048)  */
+  int32_t layers;      /* run the first n layers only; 0: all                   */
+  uint32_t eos_id;     /* generation stops before it (0xffffffff: no such id; Kimi-K2 has its own) */
+  int32_t random_init; /* do not read weights: seeded random-init of the shapes in config.json */
+  float init_sigma;    /* its standard deviation (0.02)                         */
+  uint64_t seed;
+} kx_open_options;
+typedef struct kx_model_shape {
+  char design[32];
+  int32_t n_layers, hidden, vocab, dtype, max_batch, max_context, step_tokens;
+  uint64_t weight_bytes, cache_bytes, scratch_bytes;
+} kx_model_shape;
+int kx_open_options_default(kx_open_options *opt);
+int kx_model_open(const char *dir, const kx_open_options *opt, kx_model **model);
+int kx_model_info(kx_model *model, kx_model_shape *shape);
+int kx_restart(kx_model *model, int32_t batch);
+int kx_extend(kx_model *model, const uint32_t *h_ids, int32_t n, const int32_t *h_want, int32_t n_want, float *h_logits);
+/* The residual stream (sum of the streams of a design that has several) after every layer, kept for every position
+ * while the record is on: h_out f32 [n][batch][hidden] for positions pos0 .. pos0 + n - 1.  For parity checks;
+ * Kagalorn only. */
+int kx_model_set_residual_record(kx_model *model, int on);
+int kx_model_residual(kx_model *model, int32_t layer, int32_t pos0, int32_t n, float *h_out);
 /* ---- checkpoint: runtime-index.blok -> resident weights ----------------------------------------
  * The index is the text file scripts/model_fetch.py materialize() writes (:116-131): a header line
  * `blok-runtime-index-v1`, then one line per checkpoint tensor,
