@@ -28,4 +28,4 @@ struct KxDeltaArgs {
   float *work = nullptr;          // kx_delta_work_floats(s) floats per token (not used for one position)
 };
 inline size_t kx_delta_work_floats(const KxDeltaSpec &s) { return (size_t)kx_delta_channels(s) + 2 * s.heads + s.kv_heads; }
-int kx_delta(const KxDeltaArgs &a, hipStream_t st);
+int kx_delta_launch(const KxDeltaArgs &a, hipStream_t st);

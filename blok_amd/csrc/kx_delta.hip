@@ -252,7 +252,7 @@ __global__ void __launch_bounds__(256) delta_scan_k(KxDeltaArgs a) {
 
 }  // namespace
 
-int kx_delta(const KxDeltaArgs &a, hipStream_t st) {
+int kx_delta_launch(const KxDeltaArgs &a, hipStream_t st) {
   const KxDeltaSpec &s = a.s;
   KX_REQUIRE(s.heads > 0 && s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.dim > 0 && s.vdim > 0 && s.taps > 0,
              "delta rule: heads=%d kv_heads=%d dim=%d vdim=%d taps=%d", s.heads, s.kv_heads, s.dim, s.vdim, s.taps);

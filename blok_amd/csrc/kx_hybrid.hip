@@ -82,7 +82,8 @@ struct HybridModel : kx_model {
     if (record) (void)hipFree(record);
   }
   size_t layout(char *base);
-  int fill(const std::string &dir, const kx_open_options &o);
+  int find(const std::string &dir, KxTensorMap &files) const;
+  int fill(const KxTensorMap &files, const kx_open_options &o);
   int pack(const Slot &s, const void *src, bool src_f32);
   int logits_of(const float *x, const int *map, int n, float *d_out);
 };
@@ -294,21 +295,23 @@ struct Staging {  // device memory that is gone at the end of a scope
   ~Staging() { if (p) (void)hipFree(p); }
 };
 
+// the files' tensors, each of the ones the model reads with the shape it has to have; needs no GPU
+int HybridModel::find(const std::string &dir, KxTensorMap &files) const {
+  KX_TRY(kx_safetensors_scan(dir, files));
+  for (const Slot &s : slots) {
+    const auto f = files.find(s.name);
+    KX_REQUIRE(f != files.end(), "missing tensor: %s (%s)", s.name.c_str(), dir.c_str());
+    const std::string shape = std::to_string(s.rows) + (s.cols ? "x" + std::to_string(s.cols) : "");
+    KX_REQUIRE(f->second.shape == shape && f->second.dtype != "i32", "tensor %s is %s %s, expected bf16 or f32 %s", s.name.c_str(), f->second.dtype.c_str(),
+               f->second.shape.c_str(), shape.c_str());
+  }
+  return KX_OK;
+}
+
 // The tensors from the files (or from the generator), through a staging buffer: the files have rows without padding,
 // gate and up apart, and bf16 where the arena may have f32.
-int HybridModel::fill(const std::string &dir, const kx_open_options &o) {
+int HybridModel::fill(const KxTensorMap &files, const kx_open_options &o) {
   constexpr size_t BATCH = (size_t)1 << 30;
-  KxTensorMap files;
-  if (!o.random_init) {
-    KX_TRY(kx_safetensors_scan(dir, files));
-    for (const Slot &s : slots) {
-      const auto f = files.find(s.name);
-      KX_REQUIRE(f != files.end(), "missing tensor: %s (%s)", s.name.c_str(), dir.c_str());
-      const std::string shape = std::to_string(s.rows) + (s.cols ? "x" + std::to_string(s.cols) : "");
-      KX_REQUIRE(f->second.shape == shape && f->second.dtype != "i32", "tensor %s is %s %s, expected bf16 or f32 %s", s.name.c_str(), f->second.dtype.c_str(),
-                 f->second.shape.c_str(), shape.c_str());
-    }
-  }
   auto bytes_of = [&](const Slot &s) { return ((o.random_init ? s.count() * 2 : files.at(s.name).data_bytes) + 255) & ~(size_t)255; };
   size_t most = 0;
   for (size_t i = 0; i < slots.size();) {  // the largest batch
@@ -358,7 +361,7 @@ int HybridModel::logits_of(const float *x, const int *map, int n, float *d_out) 
   g.row.w = final_norm; g.row.eps = c.eps;
   g.out = d_out;
   g.out_ld = c.vocab;
-  return kx_linear(f32, g, rows, st);
+  return kx_linear_launch(f32, g, rows, st);
 }
 
 int HybridModel::step(const uint32_t *d_ids, bool sample, int C) {
@@ -387,7 +390,7 @@ int HybridModel::step(const uint32_t *d_ids, bool sample, int C) {
     read(in, w.in, w.norm1, w.hc[0]);
     in.out = proj;
     in.out_ld = proj_ld;
-    KX_TRY(kx_linear(f32, in, rows, st));
+    KX_TRY(kx_linear_launch(f32, in, rows, st));
     write(out, w.o, w.hc[0]);
     if (l.mixer == KxHybridLayer::ATTENTION) {
       KxWindowArgs a;
@@ -396,7 +399,7 @@ int HybridModel::step(const uint32_t *d_ids, bool sample, int C) {
       a.q_norm = w.q_norm; a.k_norm = w.k_norm; a.eps = c.eps;
       a.batch = batch; a.positions = C; a.pos = pos;
       a.out = att; a.out_ld = att_ld; a.q = q; a.part = part; a.part_floats = part_floats;
-      KX_TRY(kx_window_attention(f32, a, st));
+      KX_TRY(kx_window_launch(f32, a, st));
       out.row.x = att;
       out.row.x_ld = att_ld;
     } else {
@@ -407,22 +410,22 @@ int HybridModel::step(const uint32_t *d_ids, bool sample, int C) {
       d.state = w.state; d.hist = w.hist[hist_cur]; d.hist_out = w.hist[hist_cur ^ 1];
       d.batch = batch; d.positions = C;
       d.o = delta_o; d.work = work;
-      KX_TRY(kx_delta(d, st));
+      KX_TRY(kx_delta_launch(d, st));
       out.row.kind = KX_ROW_GATED;
       out.row.o = delta_o; out.row.gate = proj + w.g_off; out.row.gate_ld = proj_ld; out.row.heads = l.delta.heads; out.row.vdim = l.delta.vdim;
       out.row.w = w.o_norm; out.row.eps = c.eps;
     }
-    KX_TRY(kx_linear(f32, out, rows, st));
+    KX_TRY(kx_linear_launch(f32, out, rows, st));
     if (l.ff) {
       KxLinArgs gu, down;
       read(gu, w.gu, w.norm2, w.hc[1]);
       gu.epi = KX_LIN_GLU;
       gu.mid = mid; gu.mid_ld = mid_ld; gu.limit = l.limit; gu.alpha = l.alpha; gu.bias = l.bias;
-      KX_TRY(kx_linear(f32, gu, rows, st));
+      KX_TRY(kx_linear_launch(f32, gu, rows, st));
       write(down, w.down, w.hc[1]);
       down.row.x = mid;
       down.row.x_ld = mid_ld;
-      KX_TRY(kx_linear(f32, down, rows, st));
+      KX_TRY(kx_linear_launch(f32, down, rows, st));
     }
     if (record) {
       hipLaunchKernelGGL(sum_streams_k, dim3(T), dim3(256), 0, st, streams, record + ((size_t)i * max_context + pos) * max_batch * W, W, S, batch, max_batch);
@@ -495,6 +498,8 @@ int hybrid_open(const char *name, const std::string &dir, const KxHybridConfig &
   m->init_sigma_ = o.init_sigma;
   auto build = [&]() -> int {
     const size_t total = m->layout(nullptr);
+    KxTensorMap files;
+    if (!o.random_init) KX_TRY(m->find(dir, files));
     size_t free_b = 0, total_b = 0;
     KX_HIP(hipMemGetInfo(&free_b, &total_b));
     KX_REQUIRE(total + ((size_t)1 << 30) <= free_b, "kx_model_open: the model needs %.1f GB of HBM, %.1f GB are free", total / 1e9, free_b / 1e9);
@@ -502,7 +507,7 @@ int hybrid_open(const char *name, const std::string &dir, const KxHybridConfig &
     KX_TRY(kx_model_resources(m, "kx_model_open"));
     KX_HIP(hipMemsetAsync(m->arena, 0, total, m->st));  // padding stays zero, cache rows that were never written are finite
     m->layout(m->arena);
-    KX_TRY(m->fill(dir, o));
+    KX_TRY(m->fill(files, o));
     KX_HIP(hipStreamSynchronize(m->st));
     return KX_OK;
   };
@@ -515,12 +520,18 @@ int hybrid_open(const char *name, const std::string &dir, const KxHybridConfig &
   return KX_OK;
 }
 
+int kagalorn_probe(const std::string &dir, const KxJson &json, kx_model_shape &shape) {
+  KxHybridConfig c;
+  KX_TRY(kx_kagalorn_config(json, c));
+  shape.n_layers = (int)c.layers.size(); shape.hidden = c.width; shape.vocab = c.vocab;
+  return KX_OK;
+}
 int kagalorn_open(const std::string &dir, const KxJson &json, const kx_open_options &o, kx_model **out) {
   KxHybridConfig c;
   KX_TRY(kx_kagalorn_config(json, c));
   return hybrid_open("Kagalorn", dir, c, o, out);
 }
 
-const KxDesignEntry entry(KxDesign{"Kagalorn", kx_kagalorn_matches, kagalorn_open});
+const KxDesignEntry entry(KxDesign{"Kagalorn", kx_kagalorn_matches, kagalorn_probe, kagalorn_open});
 
 }  // namespace

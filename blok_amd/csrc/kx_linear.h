@@ -60,4 +60,4 @@ constexpr int KX_MAX_STREAMS = 8;
 // f32: the model's type is float, else bf16.  row_buf: tokens * m.ld elements of scratch, where the rows of a step of
 // more than KX_GEMV_TOKENS tokens are built (not used for PLAIN).
 constexpr int KX_GEMV_TOKENS = 4;
-int kx_linear(bool f32, const KxLinArgs &a, void *row_buf, hipStream_t st);
+int kx_linear_launch(bool f32, const KxLinArgs &a, void *row_buf, hipStream_t st);

@@ -337,6 +337,6 @@ int linear(const KxLinArgs &a, void *row_buf, hipStream_t st) {
 
 }  // namespace
 
-int kx_linear(bool f32, const KxLinArgs &a, void *row_buf, hipStream_t st) {
+int kx_linear_launch(bool f32, const KxLinArgs &a, void *row_buf, hipStream_t st) {
   return f32 ? linear<float>(a, row_buf, st) : linear<uint16_t>(a, row_buf, st);
 }

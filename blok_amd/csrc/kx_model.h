@@ -64,6 +64,7 @@ int kx_model_resources(kx_model *m, const char *who);
 struct KxDesign {
   const char *name;
   bool (*matches)(const KxJson &config);                       // is this config.json one of the design's?
+  int (*probe)(const std::string &dir, const KxJson &config, kx_model_shape &shape);  // n_layers, hidden, vocab; no GPU
   int (*open)(const std::string &dir, const KxJson &config, const kx_open_options &o, kx_model **out);
 };
 // A design registers itself from its own file by a static object of this type, so that a program linked from some of

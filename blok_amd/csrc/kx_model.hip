@@ -744,6 +744,14 @@ bool kimi_matches(const KxJson &config) {
   return mt && mt->is(KxJson::STRING) && mt->str == "kimi_k2";
 }
 
+int kimi_probe(const std::string &dir, const KxJson &config, kx_model_shape &shape) {
+  kx_config c;
+  int rc = kx_config_default(&c);
+  if (rc || (rc = kx_index_infer_config((dir + "/runtime-index.blok").c_str(), &c))) return rc;
+  shape.n_layers = c.n_layers; shape.hidden = c.hidden; shape.vocab = c.vocab;
+  return KX_OK;
+}
+
 int kimi_open(const std::string &dir, const KxJson &config, const kx_open_options &o, kx_model **out) {
   KX_REQUIRE(o.dtype == KX_DTYPE_BF16, "kx_model_open: Kimi-K2 runs in bfloat16 only");
   KX_REQUIRE(!o.random_init, "kx_model_open: a random-init Kimi-K2 is made by kx_model_create");
@@ -758,6 +766,6 @@ int kimi_open(const std::string &dir, const KxJson &config, const kx_open_option
   return kx_model_load(&c, index.c_str(), out);
 }
 
-const KxDesignEntry entry(KxDesign{"Kimi-K2", kimi_matches, kimi_open});
+const KxDesignEntry entry(KxDesign{"Kimi-K2", kimi_matches, kimi_probe, kimi_open});
 
 }  // namespace

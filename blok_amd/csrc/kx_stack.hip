@@ -83,6 +83,22 @@ std::vector<KxDesign> &designs() {
   return d;
 }
 
+// the design that dir/config.json names
+int find_design(const std::string &dir, KxJson &config, const KxDesign **out) {
+  int rc = kx_json_file(dir + "/config.json", config);
+  if (rc) return rc;
+  std::string known;
+  for (const KxDesign &d : designs()) {
+    if (d.matches(config)) {
+      *out = &d;
+      return KX_OK;
+    }
+    known += (known.empty() ? "" : ", ") + std::string(d.name);
+  }
+  kx_set_error("%s/config.json names none of the designs here (%s)", dir.c_str(), known.c_str());
+  return KX_ERR_ARG;
+}
+
 }  // namespace
 
 KxDesignEntry::KxDesignEntry(const KxDesign &d) { designs().push_back(d); }
@@ -122,15 +138,22 @@ extern "C" int kx_model_open(const char *dir, const kx_open_options *opt, kx_mod
              "kx_model_open: max_batch=%d max_context=%d step_tokens=%d layers=%d", opt->max_batch, opt->max_context, opt->step_tokens, opt->layers);
   return kx_guard("kx_model_open", [&]() -> int {
     KxJson config;
-    int rc = kx_json_file(std::string(dir) + "/config.json", config);
+    const KxDesign *d = nullptr;
+    int rc = find_design(dir, config, &d);
+    return rc ? rc : d->open(dir, config, *opt, out);
+  });
+}
+
+extern "C" int kx_model_probe(const char *dir, kx_model_shape *out) {
+  KX_REQUIRE(dir && dir[0] && out, "kx_model_probe: null argument");
+  memset(out, 0, sizeof *out);
+  return kx_guard("kx_model_probe", [&]() -> int {
+    KxJson config;
+    const KxDesign *d = nullptr;
+    int rc = find_design(dir, config, &d);
     if (rc) return rc;
-    std::string known;
-    for (const KxDesign &d : designs()) {
-      if (d.matches(config)) return d.open(dir, config, *opt, out);
-      known += (known.empty() ? "" : ", ") + std::string(d.name);
-    }
-    kx_set_error("kx_model_open: %s/config.json names none of the designs here (%s)", dir, known.c_str());
-    return KX_ERR_ARG;
+    snprintf(out->design, sizeof out->design, "%s", d->name);
+    return d->probe(dir, config, *out);
   });
 }
 

@@ -42,4 +42,4 @@ struct KxWindowArgs {
 };
 // floats of `part` that let `tokens` tokens attend in one launch
 size_t kx_window_part_floats(const KxWindowSpec &s, int max_context, int tokens);
-int kx_window_attention(bool f32, const KxWindowArgs &a, hipStream_t st);
+int kx_window_launch(bool f32, const KxWindowArgs &a, hipStream_t st);

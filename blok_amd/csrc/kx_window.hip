@@ -499,4 +499,4 @@ size_t kx_window_part_floats(const KxWindowSpec &s, int max_context, int tokens)
   return (size_t)kx_cdiv(most_keys(s, max_context), 64) * floats_per_part(s) * tokens;
 }
 
-int kx_window_attention(bool f32, const KxWindowArgs &a, hipStream_t st) { return f32 ? attention<float>(a, st) : attention<uint16_t>(a, st); }
+int kx_window_launch(bool f32, const KxWindowArgs &a, hipStream_t st) { return f32 ? attention<float>(a, st) : attention<uint16_t>(a, st); }

@@ -50,6 +50,22 @@ class KxModelShape(C.Structure):
             (n, C.c_uint64) for n in ("weight_bytes", "cache_bytes", "scratch_bytes")]
 
 
+class KxWindowConfig(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("heads", "kv_heads", "dim", "vdim", "size", "pool", "sink", "gate")] + [
+        ("scale", C.c_float), ("eps", C.c_float)]
+
+
+class KxDeltaConfig(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("heads", "kv_heads", "dim", "vdim", "taps")] + [("unit_eps", C.c_float)]
+
+
+class KxLinearArgs(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("f32", "tokens", "rows", "cols", "ld", "row_kind", "epilogue", "streams", "groups", "heads",
+                                         "vdim", "x_ld", "gate_ld", "out_ld")] + [
+        (n, C.c_float) for n in ("eps", "limit", "alpha", "bias")] + [
+        (n, C.c_void_p) for n in ("d_w", "d_x", "d_streams_in", "d_in", "d_norm", "d_o", "d_gate", "d_mix", "d_outw", "d_out")]
+
+
 DTYPES = {"bfloat16": 0, "float32": 1}
 
 _P, _I, _U64, _F, _SZ = C.c_void_p, C.c_int32, C.c_uint64, C.c_float, C.c_size_t
@@ -119,8 +135,17 @@ _SIGS = {
     "kx_moe_decode_layer_timed": [C.POINTER(KxConfig), C.POINTER(KxMoeWeights), _P, _P, _P, _I,
                                   C.c_uint32, _P, C.POINTER(C.c_float)],
     "kx_moe_routed_only": [C.POINTER(KxConfig), C.POINTER(KxMoeWeights), _P, _P, _I, _I, _P],
+    "kx_window_create": [C.POINTER(KxWindowConfig), C.c_int, _I, _I, _I, _PP],
+    "kx_window_destroy": [_P],
+    "kx_window_run": [_P, _P, _I, _I, _I, _I, _I, _P, _P, _I, _I, _I, _P, _I, _P],
+    "kx_delta_create": [C.POINTER(KxDeltaConfig), _I, _I, _PP],
+    "kx_delta_destroy": [_P],
+    "kx_delta_restart": [_P, _P],
+    "kx_delta_run": [_P, _P, _I, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _P, _P],
+    "kx_linear_run": [C.POINTER(KxLinearArgs), _P, _P],
     "kx_open_options_default": [C.POINTER(KxOpenOptions)],
     "kx_model_open": [C.c_char_p, C.POINTER(KxOpenOptions), _PP],
+    "kx_model_probe": [C.c_char_p, C.POINTER(KxModelShape)],
     "kx_model_info": [_P, C.POINTER(KxModelShape)],
     "kx_restart": [_P, _I],
     "kx_extend": [_P, _P, _I, _P, _I, _P],

@@ -12,7 +12,7 @@ import os
 import subprocess
 from pathlib import Path
 
-from .lib import KxError, kx
+from .lib import KxError, KxModelShape, kx
 
 
 class BlokRuntimeError(RuntimeError):
@@ -142,7 +142,7 @@ def executor_path():
     return Path(os.getenv("BLOK_KIMI_EXEC_BIN", Path(__file__).parent / "kx-kimi-exec"))
 
 
-def _run_executor(argv, max_time):
+def _run_executor(argv, max_time, vocab=KIMI_TEXT["vocab_size"]):
     """The executor's token ids: one JSON line on stdout, a non-zero exit code means failure with the reason on
     stderr (src/kimi_exec.cu:495-498, :901-903)."""
     try:
@@ -156,7 +156,6 @@ def _run_executor(argv, max_time):
     except json.JSONDecodeError as error:
         raise BlokRuntimeError(f"executor returned invalid JSON: {done.stdout!r}") from error
     ids = report.get("token_ids") if report.get("status") == "ok" else None
-    vocab = KIMI_TEXT["vocab_size"]
     if not isinstance(ids, list) or any(type(i) is not int or not 0 <= i < vocab for i in ids):
         raise BlokRuntimeError(f"executor failed: {report}")
     return ids
@@ -181,6 +180,20 @@ def generate(*, model_dir, prompt, max_tokens, max_time):
     if layers:
         argv += ["--layers", layers]
     return encoding.decode(_run_executor(argv, max_time))
+
+
+def generate_ids(*, model_dir, prompt_ids, max_tokens, max_time, dtype="bfloat16", eos_id=None):
+    """Greedy token ids after `prompt_ids` from a model directory of any design the library's registry knows
+    (kx_model_open); such a directory needs no tokenizer."""
+    if not prompt_ids or max_tokens <= 0 or max_time <= 0:
+        raise BlokRuntimeError("prompt must be non-empty and limits must be positive")
+    shape = KxModelShape()
+    if kx().kx_model_probe(str(model_dir).encode(), C.byref(shape)) != 0:
+        raise BlokRuntimeError(kx().kx_last_error().decode("utf-8", "replace"))
+    argv = [str(executor_path()), "--model", str(model_dir), "--dtype", dtype, "--prompt-tokens", ",".join(map(str, prompt_ids)),
+            "--tokens", str(max_tokens)]
+    argv += ["--ignore-eos"] if eos_id is None else ["--eos", str(eos_id)]
+    return _run_executor(argv, max_time, shape.vocab)
 
 
 def answer(text):

@@ -266,6 +266,53 @@ int kx_decode_step(kx_model *model, const uint32_t *h_ids);
 int kx_greedy_sample(kx_model *model, uint32_t *h_out);
 int kx_generate(kx_model *model, const uint32_t *h_prompt, int32_t batch, int32_t prompt_len,
                 int32_t n_tokens, int ignore_eos, uint32_t *h_out, int32_t *h_counts);
+/* ---- operators of the hybrid decoder ---------------------------------------------------------
+ * The mechanisms of the Kagalorn design on their own; the model's steps run the same kernels.  f32: 1 for 32-bit weights
+ * and activation rows (float), 0 for bf16; everything else is float.  Token i * batch + b is position pos + i of
+ * sequence b.  No counterparts in the reference.
+ *
+ * kx_window_*: grouped-query attention over a sliding window and pooled blocks.  Position i sees the positions j with
+ *   0 <= i - j < size and, as one key and value each, the blocks [b pool, (b + 1) pool) that end at or before i - size:
+ *   the means of their cached keys and values (pool 0: none).  A kx_window holds the cache and scratch of one layer.
+ *   d_proj f32 [tokens][proj_ld]: q [heads][dim], k [kv_heads][dim], v [kv_heads][vdim] and, with `gate`, the output
+ *   gate's pre-activation [heads][vdim], each from the given column on.  d_q_norm / d_k_norm: weights of an RMS norm over
+ *   the whole q (k) row, or NULL.  d_out [tokens][out_ld] of the number format.
+ * kx_delta_*: the gated delta rule behind short causal convolutions with silu.  d_proj f32 [tokens][proj_ld] holds q, k
+ *   [kv_heads][dim], v [heads][vdim] and the projections of step size and decay, b and a [heads].  d_conv f32 [channels][taps]
+ *   (q, k, v channels in turn); d_o f32 [tokens][heads * vdim].  A kx_delta holds state and convolution inputs.
+ * kx_linear_run: y = W row with the row built from residual streams (row_kind 1: w * groupnorm(sum_s in[s] x_s)), from the
+ *   delta rule's read-out (row_kind 2: per head rms norm * w * silu(gate)) or taken from memory (0), and the product stored
+ *   (epilogue 0), made into a clamped gated activation (1; W's rows are blocks of 32 gate rows and their 32 up rows), or
+ *   written to all streams (2: x_t <- sum_s mix[s][t] x_s + outw[t] y).  Matrices have rows of `ld` elements, a multiple of
+ *   64, zero beyond `cols`; rows in memory (x, mid) likewise.                                                            */
+typedef struct kx_window_config {
+  int32_t heads, kv_heads, dim, vdim, size, pool, sink, gate;
+  float scale, eps;
+} kx_window_config;
+typedef struct kx_window kx_window;
+int kx_window_create(const kx_window_config *cfg, int f32, int32_t max_batch, int32_t max_context, int32_t max_positions, kx_window **out);
+int kx_window_destroy(kx_window *w);
+int kx_window_run(kx_window *w, const void *d_proj, int32_t proj_ld, int32_t q_off, int32_t k_off, int32_t v_off, int32_t g_off,
+                  const void *d_q_norm, const void *d_k_norm, int32_t batch, int32_t positions, int32_t pos, void *d_out,
+                  int32_t out_ld, void *stream);
+typedef struct kx_delta_config {
+  int32_t heads, kv_heads, dim, vdim, taps;
+  float unit_eps; /* under the root of the unit norms of q and k */
+} kx_delta_config;
+typedef struct kx_delta kx_delta;
+int kx_delta_create(const kx_delta_config *cfg, int32_t max_batch, int32_t max_positions, kx_delta **out);
+int kx_delta_destroy(kx_delta *d);
+int kx_delta_restart(kx_delta *d, void *stream);
+int kx_delta_run(kx_delta *d, const void *d_proj, int32_t proj_ld, int32_t q_off, int32_t k_off, int32_t v_off, int32_t b_off,
+                 int32_t a_off, const void *d_conv, const void *d_a_log, const void *d_dt_bias, int32_t batch, int32_t positions,
+                 void *d_o, void *stream);
+typedef struct kx_linear_args {
+  int32_t f32, tokens, rows, cols, ld, row_kind, epilogue, streams, groups, heads, vdim, x_ld, gate_ld, out_ld;
+  float eps, limit, alpha, bias;
+  const void *d_w, *d_x, *d_streams_in, *d_in, *d_norm, *d_o, *d_gate, *d_mix, *d_outw;
+  void *d_out; /* epilogue 0: f32 [tokens][out_ld]; 1: [tokens][out_ld] of the format; 2: f32 [tokens][streams][rows], in place */
+} kx_linear_args;
+int kx_linear_run(const kx_linear_args *args, void *d_row_scratch, void *stream); /* scratch: tokens * ld elements of the format */
 /* ---- model directories ---------------------------------------------------------------------
  * kx_model_open  : reads <dir>/config.json, finds the design it names in the library's registry and opens the model
  *                  with it.  Two designs are known: Kimi-K2 (config.json of the checkpoint with runtime-index.blok
@@ -273,6 +320,8 @@ int kx_generate(kx_model *model, const uint32_t *h_prompt, int32_t batch, int32_
  *                  Every kx_model entry point works on the result; those that set up a mechanism only Kimi-K2 has
  *                  (kx_model_set_fusion, _set_exact, _set_attention_kernel, routing, latent cache rows) return an error
  *                  on another design.
+ * kx_model_probe : design, n_layers, hidden and vocab of a model directory, from its configuration alone (no GPU; the
+ *                  other fields are 0).
  * kx_model_info  : the opened model's shape.
  * kx_restart     : forgets the sequences; the next kx_extend starts `batch` new ones at position 0.
  * kx_extend      : appends n positions to every sequence; h_ids u32 [batch][n].  The positions are run in steps of up
@@ -299,6 +348,7 @@ typedef struct kx_model_shape {
 } kx_model_shape;
 int kx_open_options_default(kx_open_options *opt);
 int kx_model_open(const char *dir, const kx_open_options *opt, kx_model **model);
+int kx_model_probe(const char *dir, kx_model_shape *shape);
 int kx_model_info(kx_model *model, kx_model_shape *shape);
 int kx_restart(kx_model *model, int32_t batch);
 int kx_extend(kx_model *model, const uint32_t *h_ids, int32_t n, const int32_t *h_want, int32_t n_want, float *h_logits);
