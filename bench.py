@@ -11,6 +11,8 @@ already resident in HBM.  Workloads:
   moe_layer : config 2 alone, one routed-MoE decode layer at Kimi-K2 shape for `--tokens`
               tokens.  Weights of several independent layers are cycled so that neither L2
               nor the 256 MB Infinity Cache can serve them.
+  hybrid    : the Kagalorn design at the layer sizes of real models (random weights), prefill and decode, each beside a
+              Kimi-K2 stack of dense layers of the same hidden size, heads and feed-forward.
 Prints ONE JSON line.
 """
 import argparse
@@ -691,12 +693,116 @@ def run_load(args):
           flush=True)
 
 
+# layers of the hybrid workload: attention and delta rule in turn, sizes of models of about 1, 8 and 70 billion parameters
+HYBRID_SIZES = {"w2048": (2048, 16, 4, 8192), "w4096": (4096, 32, 8, 12288), "w8192": (8192, 64, 8, 28672)}   # width, heads, kv_heads, ff
+HYBRID_LAYERS, HYBRID_VOCAB, HYBRID_DIM, HYBRID_WINDOW, HYBRID_POOL = 8, 32768, 128, 1024, 16
+
+
+def hybrid_config(size):
+    width, heads, kv, ff = HYBRID_SIZES[size]
+    mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
+    attn = {"type": "attention", "mlp": mlp, "mixer": {"heads": heads, "kv_heads": kv, "dim": HYBRID_DIM, "vdim": HYBRID_DIM, "scale": HYBRID_DIM ** -0.5,
+                                                       "mask": {"size": HYBRID_WINDOW, "pool": HYBRID_POOL}}}
+    delta = {"type": "delta", "mlp": mlp, "mixer": {"heads": heads, "kv_heads": heads // 2, "dim": HYBRID_DIM, "vdim": HYBRID_DIM, "conv": 4}}
+    return {"architecture": "Kagalorn", "vocab": HYBRID_VOCAB, "width": width, "streams": 2, "norm": {"eps": 1e-5, "groups": 2},
+            "layers": [attn, delta] * (HYBRID_LAYERS // 2)}
+
+
+def timed_model(lib, model, prompt, P, chunk, K, W, vocab):
+    """ms per prefill of a P-token prompt and per decode step after it (batch 1, greedy, ids stay on the device); the best of
+    three prefills, so that the first one's code loading does not count."""
+    from blok_amd.lib import check
+    st = C.c_void_p()
+    check(lib.kx_model_stream(model, C.byref(st)))
+    check(lib.kx_model_set_prefill_chunk(model, chunk))
+    e = [C.c_void_p() for _ in range(2)]
+    for ev in e:
+        check(lib.kx_event_create(C.byref(ev)))
+    ms, pre = C.c_float(), []
+    for _ in range(3):
+        check(lib.kx_event_record(e[0], st))
+        check(lib.kx_prefill(model, prompt.ctypes.data, 1, P))
+        check(lib.kx_event_record(e[1], st))
+        check(lib.kx_event_elapsed_ms(e[0], e[1], C.byref(ms)))
+        pre.append(ms.value)
+    for _ in range(W):
+        check(lib.kx_decode_step(model, None))
+    check(lib.kx_event_record(e[0], st))
+    for _ in range(K):
+        check(lib.kx_decode_step(model, None))
+    check(lib.kx_event_record(e[1], st))
+    check(lib.kx_event_elapsed_ms(e[0], e[1], C.byref(ms)))
+    for ev in e:
+        check(lib.kx_event_destroy(ev))
+    return min(pre), ms.value / K
+
+
+def hybrid_leg(lib, size, design, P, K, W, seed, chunk):
+    import tempfile
+    from blok_amd.lib import KxOpenOptions, check, default_config
+    width, heads, kv, ff = HYBRID_SIZES[size]
+    model = C.c_void_p()
+    if design == "kagalorn":
+        o = KxOpenOptions()
+        check(lib.kx_open_options_default(C.byref(o)))
+        o.max_context, o.random_init, o.seed, o.step_tokens = P + K + W + 1, 1, seed, chunk
+        with tempfile.TemporaryDirectory() as d:
+            with open(os.path.join(d, "config.json"), "w") as f:
+                json.dump(hybrid_config(size), f)
+            check(lib.kx_model_open(d.encode(), C.byref(o), C.byref(model)))
+        hd = heads * HYBRID_DIM
+        attn = width * (hd + 2 * kv * HYBRID_DIM + hd + hd)              # q, k, v, gate, output
+        delta = width * (2 * (heads // 2) * HYBRID_DIM + 3 * hd + 2 * heads)
+        layer = [attn, delta] * (HYBRID_LAYERS // 2)
+        keys = HYBRID_WINDOW + max(0, P - HYBRID_WINDOW) // HYBRID_POOL
+        state = HYBRID_LAYERS // 2 * (keys * kv * 2 * HYBRID_DIM * 2 + heads * HYBRID_DIM * HYBRID_DIM * 4 * 2)   # cache rows read, state read and written
+    else:
+        c = default_config()
+        c.n_layers = c.first_dense = HYBRID_LAYERS
+        c.hidden, c.heads, c.dense_inter, c.vocab, c.max_context, c.seed = width, heads, ff, HYBRID_VOCAB, P + K + W + 1, seed
+        check(lib.kx_model_create(C.byref(c), C.byref(model)))
+        kva = c.kv_rank + c.qk_rope
+        layer = [width * (c.q_rank + kva) + heads * (c.qk_nope + c.qk_rope) * c.q_rank + heads * (c.qk_nope + c.v_head) * c.kv_rank
+                 + width * heads * c.v_head] * HYBRID_LAYERS
+        state = HYBRID_LAYERS * P * kva * 2
+    params = sum(layer) + HYBRID_LAYERS * 3 * ff * width
+    prompt = device_tokens(lib, P, seed, HYBRID_VOCAB)
+    pre, dec = timed_model(lib, model, prompt, P, chunk, K, W, HYBRID_VOCAB)
+    check(lib.kx_model_destroy(model))
+    read = 2 * (params + HYBRID_VOCAB * width) + state
+    flop = 2.0 * P * params
+    return {"prefill_tok_s": round(P * 1e3 / pre, 1), "prefill_ms": round(pre, 3), "prefill_tflops_of_the_products": round(flop / pre / 1e9, 1),
+            "prefill_frac_of_mfma_peak": round(flop / pre / 1e9 / 2500, 4), "decode_tok_s": round(1e3 / dec, 1), "decode_ms": round(dec, 4),
+            "decode_bytes": int(read), "decode_frac_of_hbm_peak": round(read / dec / 1e6 / HBM_PEAK_GBS, 4)}
+
+
+def run_hybrid(args):
+    from blok_amd.lib import check, kx
+    lib = kx()
+    name = C.create_string_buffer(256)
+    check(lib.kx_device_info(name, 256, None, None))
+    P = args.prompt if args.prompt != 1024 else 4096
+    K = args.steps if args.steps != 256 else 64
+    chunk = args.prefill_chunk if args.prefill_chunk > 1 else 2048
+    sizes = {}
+    for size in (args.hybrid_size.split(",") if args.hybrid_size else HYBRID_SIZES):
+        sizes[size] = {d: hybrid_leg(lib, size, d, P, K, args.warmup, args.seed, chunk) for d in args.hybrid_designs.split(",")}
+        print(f"{size}: {sizes[size]}", file=sys.stderr, flush=True)
+    last = list(sizes)[-1]
+    print(json.dumps({"metric": "hybrid decoder, decode tok/s at batch 1", "value": list(sizes[last].values())[0]["decode_tok_s"], "unit": "tok/s", "n_gpus": 1,
+                      "steps": K, "warmup": args.warmup, "higher_is_better": True, "dtype": "bf16", "data": "synthetic", "device": name.value.decode(),
+                      "config": {"layers": HYBRID_LAYERS, "vocab": HYBRID_VOCAB, "prompt": P, "positions_per_prefill_step": chunk, "sizes": HYBRID_SIZES,
+                                 "window": HYBRID_WINDOW, "pool": HYBRID_POOL}, "sizes": sizes}), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=256)
     ap.add_argument("--warmup", type=int, default=8)
-    ap.add_argument("--workload", default="stack", choices=["stack", "moe_layer", "prefill", "mla", "copy", "load"])
+    ap.add_argument("--workload", default="stack", choices=["stack", "moe_layer", "prefill", "mla", "copy", "load", "hybrid"])
+    ap.add_argument("--hybrid-size", default=None, help="hybrid: sizes to run, with commas (default: all)")
+    ap.add_argument("--hybrid-designs", default="kagalorn,kimi_dense", help="hybrid: designs to run")
     ap.add_argument("--load-dir", default=None, help="where the load workload writes its sparse shards (default: the temp dir)")
     ap.add_argument("--context", type=int, default=32768)
     ap.add_argument("--copy-mib", type=int, default=1024)
@@ -729,6 +835,9 @@ def main():
         return
     if args.workload == "mla":
         run_mla(args)
+        return
+    if args.workload == "hybrid":
+        run_hybrid(args)
         return
     if args.workload == "prefill":
         if args.tokens == 1:

@@ -25,7 +25,14 @@ struct KxDeltaArgs {
   float *hist_out = nullptr;      // the same after this step (another buffer)
   int batch = 0, positions = 0;   // token i * batch + b is the i-th new position of sequence b
   float *o = nullptr;             // f32 [tokens][heads * vdim]
-  float *work = nullptr;          // kx_delta_work_floats(s) floats per token (not used for one position)
+  float *work = nullptr;          // kx_delta_work_floats(s, batch, positions) floats (not used for one position)
 };
-inline size_t kx_delta_work_floats(const KxDeltaSpec &s) { return (size_t)kx_delta_channels(s) + 2 * s.heads + s.kv_heads; }
+// Tokens go through the state in blocks of KX_DELTA_BLOCK; per token and head there are KX_DELTA_COEF numbers.
+constexpr int KX_DELTA_BLOCK = 4, KX_DELTA_COEF = 12;
+// keys and queries lie in the scratch with rows of 32, 64, 128 or 256
+__host__ __device__ inline int kx_delta_row(const KxDeltaSpec &s) { return s.dim <= 32 ? 32 : s.dim <= 64 ? 64 : s.dim <= 128 ? 128 : 256; }
+inline size_t kx_delta_work_floats(const KxDeltaSpec &s, int batch, int positions) {
+  const size_t padded = (size_t)batch * ((positions + KX_DELTA_BLOCK - 1) / KX_DELTA_BLOCK * KX_DELTA_BLOCK);
+  return padded * ((size_t)KX_DELTA_COEF * s.heads + kx_delta_channels(s) + 2 * s.kv_heads * kx_delta_row(s));
+}
 int kx_delta_launch(const KxDeltaArgs &a, hipStream_t st);

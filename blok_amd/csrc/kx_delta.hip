@@ -2,11 +2,19 @@
 //
 // One token per sequence: delta_step_k.  A workgroup owns 32 columns of one head's state; it convolves and norms the
 // head's q and k itself, reads its columns once, and writes them once.
-// Several positions: delta_prep_k (convolutions, unit norms, beta, decay; tokens in parallel), delta_hist_k (the
-// convolutions' inputs that the next step needs) and delta_scan_k, which keeps the state in registers: the columns of
-// a head's state do not meet, so a column is spread over dim / 8 lanes with 8 rows each, and a wave goes through the
-// tokens with two sums over those lanes per token, S^T k and S^T q; the read-out after the write is
-// g S^T q + u (k . q).
+//
+// Several positions: delta_conv_k (convolutions and silu), delta_unit_k (unit norms and the numbers below),
+// delta_hist_k (the convolutions' inputs that the next step needs) and delta_scan_k, which keeps the state in registers:
+// the columns of a head's state do not meet, so a column is spread over dim / 8 lanes with 8 rows each, and a wave goes
+// through the tokens.  It takes them in blocks of four, so that the sums over a column's lanes do not wait for each
+// other: with S the state before the block, D(i, j) the product of the decays of tokens i + 1 .. j and D(j) that of tokens
+// 1 .. j of the block,
+//   u_j = beta_j (v_j - D(j) S^T k_j - sum_{i < j} D(i, j) (k_i . k_j) u_i)
+//   o_j = D(j) S^T q_j + sum_{i <= j} D(i, j) (k_i . q_j) u_i
+//   S  <- D(4) S + sum_i D(i, 4) k_i u_i^T,
+// which is the recurrence written out for four tokens.  The numbers that do not depend on the column -- per token D(j),
+// beta, D(j, 4), D(j - d, j) (k_{j-d} . k_j) for d = 1..3 and D(j - d, j) (k_{j-d} . q_j) for d = 0..3 -- are made
+// once per head by delta_unit_k and come to the scan through scalar loads.
 #include <algorithm>
 #include <atomic>
 #include "kx_common.h"
@@ -102,49 +110,120 @@ __global__ void __launch_bounds__(256) delta_step_k(KxDeltaArgs a) {
   }
 }
 
-// work, per token: q [kv_heads * dim], k, v [heads * vdim], decay and beta [heads], k . q [kv_heads]
+constexpr int NB = KX_DELTA_BLOCK, NCF = KX_DELTA_COEF;
+enum { CF_GAMMA = 0, CF_BETA = 1, CF_END = 2, CF_KK = 3, CF_KQ = 6 };  // places of a token's numbers
+
 struct Work {
-  float *qkv, *gb, *kq;
+  float *coef;  // [batch][heads][padded positions][NCF]
+  float *qk;    // [tokens][kv_heads][2][kx_delta_row]: unit k, unit q times dim^-1/2, zeros behind them
+  float *raw;   // [tokens][channels]: q, k, v behind convolution and silu
+  int padded;
 };
-__device__ __forceinline__ Work work_of(const KxDeltaArgs &a) {
-  const size_t T = (size_t)a.batch * a.positions;
+__host__ __device__ __forceinline__ Work work_of(const KxDeltaArgs &a) {
   Work w;
-  w.qkv = a.work;
-  w.gb = w.qkv + T * kx_delta_channels(a.s);
-  w.kq = w.gb + T * 2 * a.s.heads;
+  w.padded = (a.positions + NB - 1) / NB * NB;
+  w.coef = a.work;
+  w.qk = w.coef + (size_t)a.batch * a.s.heads * w.padded * NCF;
+  w.raw = w.qk + (size_t)a.batch * a.positions * a.s.kv_heads * 2 * kx_delta_row(a.s);
   return w;
 }
 
-__global__ void __launch_bounds__(256) delta_prep_k(KxDeltaArgs a) {
-  const KxDeltaSpec &s = a.s;
-  const int tok = blockIdx.x, i = tok / a.batch, b = tok - i * a.batch, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int D = s.dim, nq = s.kv_heads * D, C = kx_delta_channels(s);
-  const Work w = work_of(a);
-  float *out = w.qkv + (size_t)tok * C;
-  const float *pr = a.proj + (size_t)tok * a.proj_ld;
-  for (int h = wave; h < s.kv_heads; h += 4) {
-    float qq = 0.0f, kk = 0.0f, kq = 0.0f;
-    for (int d = lane; d < D; d += 64) {
-      const float q = conv_silu(a, b, i, h * D + d), k = conv_silu(a, b, i, nq + h * D + d);
-      qq = __builtin_fmaf(q, q, qq);
-      kk = __builtin_fmaf(k, k, kk);
-      kq = __builtin_fmaf(k, q, kq);
-      out[h * D + d] = q;  // this lane's own words, scaled below
-      out[nq + h * D + d] = k;
+constexpr int CONV_TOKENS = 16;  // positions a thread of delta_conv_k goes through
+template <int TAPS>              // 0: any number
+__global__ void __launch_bounds__(256) delta_conv_k(KxDeltaArgs a) {
+  const int C = kx_delta_channels(a.s), ch = blockIdx.x * 256 + threadIdx.x, b = blockIdx.z;
+  const int i0 = blockIdx.y * CONV_TOKENS, i1 = min(i0 + CONV_TOKENS, a.positions);
+  if (ch >= C) return;
+  float *raw = work_of(a).raw;
+  if constexpr (TAPS == 0) {
+    for (int i = i0; i < i1; ++i) raw[(size_t)(i * a.batch + b) * C + ch] = conv_silu(a, b, i, ch);
+  } else {
+    const int off = channel_off(a, ch);
+    float w[TAPS], x[CONV_TOKENS + TAPS - 1];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[j] = a.conv[(size_t)ch * TAPS + j];
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j) x[j] = conv_input(a, b, i0 - (TAPS - 1) + j, ch, off);
+#pragma unroll
+    for (int j = 0; j < CONV_TOKENS; ++j) x[TAPS - 1 + j] = a.proj[(size_t)(min(i0 + j, a.positions - 1) * a.batch + b) * a.proj_ld + off];
+#pragma unroll
+    for (int j = 0; j < CONV_TOKENS; ++j) {
+      float v = 0.0f;
+#pragma unroll
+      for (int t = 0; t < TAPS; ++t) v = __builtin_fmaf(w[t], x[j + t], v);
+      if (i0 + j < i1) raw[(size_t)((i0 + j) * a.batch + b) * C + ch] = kx_siluf(v);
     }
-    qq = kx_rsqrtf(kxr::wave_sum(qq) + s.unit_eps) * kx_rsqrtf((float)D);
-    kk = kx_rsqrtf(kxr::wave_sum(kk) + s.unit_eps);
-    kq = kxr::wave_sum(kq) * qq * kk;
-    for (int d = lane; d < D; d += 64) {
-      out[h * D + d] *= qq;
-      out[nq + h * D + d] *= kk;
-    }
-    if (lane == 0) w.kq[(size_t)tok * s.kv_heads + h] = kq;
   }
-  for (int x = threadIdx.x; x < s.heads * s.vdim; x += 256) out[2 * nq + x] = conv_silu(a, b, i, 2 * nq + x);
-  for (int h = threadIdx.x; h < s.heads; h += 256) {
-    w.gb[((size_t)tok * s.heads + h) * 2] = decay_of(a, pr, h);
-    w.gb[((size_t)tok * s.heads + h) * 2 + 1] = kx_sigmoidf(pr[a.b_off + h]);
+}
+
+// one wave per (position, key head)
+__global__ void __launch_bounds__(256) delta_unit_k(KxDeltaArgs a) {
+  const KxDeltaSpec &s = a.s;
+  const int lane = threadIdx.x & 63, D = s.dim, nq = s.kv_heads * D, C = kx_delta_channels(s), ratio = s.heads / s.kv_heads;
+  const Work w = work_of(a);
+  const int item = blockIdx.x * 4 + (threadIdx.x >> 6), kvh = item % s.kv_heads, i = item / s.kv_heads, b = blockIdx.y;
+  if (i >= w.padded) return;
+  const int j = i % NB, t0 = i - j;  // place in the block, and the block's first position
+  float dot[NB + NB - 1] = {}, inv[NB] = {};  // kk of d = 1.., kq of d = 0..
+  if (i < a.positions) {
+    const float *row[NB];
+#pragma unroll
+    for (int d = 0; d < NB; ++d) row[d] = w.raw + (size_t)((i - min(d, j)) * a.batch + b) * C + kvh * D;
+    float qq = 0.0f, ss[NB] = {};
+    for (int x = lane; x < D; x += 64) {
+      const float q = row[0][x];
+      float k[NB];
+#pragma unroll
+      for (int d = 0; d < NB; ++d) k[d] = row[d][nq + x];
+      qq = __builtin_fmaf(q, q, qq);
+#pragma unroll
+      for (int d = 0; d < NB; ++d) {
+        ss[d] = __builtin_fmaf(k[d], k[d], ss[d]);
+        dot[NB - 1 + d] = __builtin_fmaf(k[d], q, dot[NB - 1 + d]);
+        if (d) dot[d - 1] = __builtin_fmaf(k[d], k[0], dot[d - 1]);
+      }
+    }
+    const float qsc = kx_rsqrtf(kxr::wave_sum(qq) + s.unit_eps) * kx_rsqrtf((float)D);
+#pragma unroll
+    for (int d = 0; d < NB; ++d) inv[d] = kx_rsqrtf(kxr::wave_sum(ss[d]) + s.unit_eps);
+#pragma unroll
+    for (int d = 0; d < NB; ++d) {
+      dot[NB - 1 + d] = kxr::wave_sum(dot[NB - 1 + d]) * inv[d] * qsc;
+      if (d) dot[d - 1] = kxr::wave_sum(dot[d - 1]) * inv[d] * inv[0];
+    }
+    const int DP = kx_delta_row(s);
+    float *out = w.qk + ((size_t)(i * a.batch + b) * s.kv_heads + kvh) * 2 * DP;
+    for (int x = lane; x < DP; x += 64) {
+      out[x] = x < D ? row[0][nq + x] * inv[0] : 0.0f;
+      out[DP + x] = x < D ? row[0][x] * qsc : 0.0f;
+    }
+  }
+  for (int r = lane; r < ratio; r += 64) {  // the heads that share the key
+    const int h = kvh * ratio + r;
+    float g[NB];  // decays of the block; a position past the end leaves the state as it is
+#pragma unroll
+    for (int d = 0; d < NB; ++d)
+      g[d] = t0 + d < a.positions ? decay_of(a, a.proj + (size_t)((t0 + d) * a.batch + b) * a.proj_ld, h) : 1.0f;
+    float *cf = w.coef + (((size_t)b * s.heads + h) * w.padded + i) * NCF;
+    float gamma = 1.0f, end = 1.0f;
+#pragma unroll
+    for (int d = 0; d < NB; ++d) {
+      if (d <= j) gamma *= g[d];
+      else end *= g[d];
+    }
+    cf[CF_GAMMA] = gamma;
+    cf[CF_BETA] = i < a.positions ? kx_sigmoidf(a.proj[(size_t)(i * a.batch + b) * a.proj_ld + a.b_off + h]) : 0.0f;
+    cf[CF_END] = end;
+    float down = 1.0f;  // D(j - d, j)
+#pragma unroll
+    for (int d = 0; d < NB; ++d) {
+      const bool in = d <= j;  // the other token is in the block
+      cf[CF_KQ + d] = in ? down * dot[NB - 1 + d] : 0.0f;
+      if (d) cf[CF_KK + d - 1] = in ? down * dot[d - 1] : 0.0f;
+#pragma unroll
+      for (int x = 0; x < NB; ++x)
+        if (x == j - d) down *= g[x];
+    }
   }
 }
 
@@ -170,77 +249,117 @@ __device__ __forceinline__ float column_sum(float v) {  // over the LPC lanes of
   return v;
 }
 
+// A block's numbers, through the scalar cache: they are the same for the whole workgroup and this kernel does not write them.
+typedef const __attribute__((address_space(4))) float *ScalarPtr;
+struct Coefs {
+  float v[NB][NCF];
+  __device__ __forceinline__ void load(const float *p) {
+    const ScalarPtr q = (ScalarPtr)p;
+#pragma unroll
+    for (int j = 0; j < NB; ++j)
+#pragma unroll
+      for (int x = 0; x < NCF; ++x) v[j][x] = q[j * NCF + x];
+  }
+};
+
 template <int LPC>  // lanes per column, 8 rows of the state each
 __global__ void __launch_bounds__(256) delta_scan_k(KxDeltaArgs a) {
   constexpr int DP = LPC * 8, COLS = 256 / LPC, CT = LPC >= 16 ? 16 : 32;  // CT: tokens per staged block
   __shared__ __attribute__((aligned(16))) float kq_s[2][CT][2][DP];
   __shared__ float v_s[2][CT][COLS];
-  __shared__ float sc_s[2][CT][4];  // decay, beta, k . q
   const KxDeltaSpec &s = a.s;
   const int D = s.dim, V = s.vdim, tid = threadIdx.x;
   const int h = blockIdx.y, b = blockIdx.z, c0 = blockIdx.x * COLS, kvh = h / (s.heads / s.kv_heads), nq = s.kv_heads * D;
   const int C = kx_delta_channels(s), r0 = (tid % LPC) * 8, cl = tid / LPC, col = c0 + cl, n = a.positions;
   const Work w = work_of(a);
+  const float *coef = w.coef + ((size_t)b * s.heads + h) * w.padded * NCF;
   float *st = a.state + ((size_t)b * s.heads + h) * D * V;
   float S[8];
 #pragma unroll
   for (int r = 0; r < 8; ++r) S[r] = r0 + r < D && col < V ? st[(size_t)(r0 + r) * V + col] : 0.0f;
-  // A block of tokens goes through registers into one of two LDS stages while the other is worked on.  Places past the
-  // last token hold a token that leaves the state as it is.
-  constexpr int NK = CT * DP * 2 / 256, NV = (CT * COLS + 255) / 256;
-  float rk[NK], rv[NV], rs = 0.0f;
+  // A stage of tokens goes through registers into one of two LDS stages while the other is worked on.  Places past the last
+  // token repeat it: their numbers in `coef` make them leave the state alone.
+  constexpr int NK = CT * DP * 2 / 4 / 256, NV = (CT * COLS + 255) / 256;
+  float4 rk[NK];
+  float rv[NV];
   auto fetch = [&](int t0) {
 #pragma unroll
     for (int x = 0; x < NK; ++x) {
-      const int at = x * 256 + tid, d = at % DP, q = at / DP & 1, t = t0 + at / (2 * DP);
-      rk[x] = t < n && d < D ? w.qkv[(size_t)(t * a.batch + b) * C + (q ? 0 : nq) + kvh * D + d] : 0.0f;
+      const int at = (x * 256 + tid) * 4, t = min(t0 + at / (2 * DP), n - 1);
+      rk[x] = *(const float4 *)(w.qk + ((size_t)(t * a.batch + b) * s.kv_heads + kvh) * 2 * DP + at % (2 * DP));
     }
 #pragma unroll
     for (int x = 0; x < NV; ++x) {
-      const int at = x * 256 + tid, t = t0 + at / COLS, cc = c0 + at % COLS;
-      rv[x] = t < n && cc < V && at < CT * COLS ? w.qkv[(size_t)(t * a.batch + b) * C + 2 * nq + h * V + cc] : 0.0f;
-    }
-    if (tid < CT * 3) {
-      const int t = t0 + tid / 3, f = tid % 3;
-      rs = t >= n ? (f == 0 ? 1.0f : 0.0f) : f < 2 ? w.gb[((size_t)(t * a.batch + b) * s.heads + h) * 2 + f] : w.kq[(size_t)(t * a.batch + b) * s.kv_heads + kvh];
+      const int at = min(x * 256 + tid, CT * COLS - 1), t = min(t0 + at / COLS, n - 1), cc = min(c0 + at % COLS, V - 1);
+      rv[x] = w.raw[(size_t)(t * a.batch + b) * C + 2 * nq + h * V + cc];
     }
   };
   auto put = [&](int stage) {
 #pragma unroll
-    for (int x = 0; x < NK; ++x) {
-      const int at = x * 256 + tid;
-      kq_s[stage][at / (2 * DP)][at / DP & 1][at % DP] = rk[x];
-    }
+    for (int x = 0; x < NK; ++x) *(float4 *)(&kq_s[stage][0][0][0] + (x * 256 + tid) * 4) = rk[x];
 #pragma unroll
     for (int x = 0; x < NV; ++x) {
       const int at = x * 256 + tid;
       if (at < CT * COLS) v_s[stage][at / COLS][at % COLS] = rv[x];
     }
-    if (tid < CT * 3) sc_s[stage][tid / 3][tid % 3] = rs;
   };
+  Coefs cf[2];
+  cf[0].load(coef);
   fetch(0);
   put(0);
   __syncthreads();
   for (int t0 = 0, stage = 0; t0 < n; t0 += CT, stage ^= 1) {
     if (t0 + CT < n) fetch(t0 + CT);
-#pragma unroll 4
-    for (int t = 0; t < CT; ++t) {
-      const float *kp = &kq_s[stage][t][0][r0], *qp = &kq_s[stage][t][1][r0];
-      const float4 ka = *(const float4 *)kp, kb = *(const float4 *)(kp + 4), qa = *(const float4 *)qp, qb = *(const float4 *)(qp + 4);
-      const float k[8] = {ka.x, ka.y, ka.z, ka.w, kb.x, kb.y, kb.z, kb.w}, q[8] = {qa.x, qa.y, qa.z, qa.w, qb.x, qb.y, qb.z, qb.w};
-      const float g = sc_s[stage][t][0], beta = sc_s[stage][t][1], kq = sc_s[stage][t][2];
-      float sk = 0.0f, sq = 0.0f;
 #pragma unroll
-      for (int r = 0; r < 8; ++r) {
-        sk = __builtin_fmaf(S[r], k[r], sk);
-        sq = __builtin_fmaf(S[r], q[r], sq);
+    for (int tb = 0; tb < CT; tb += NB) {
+      if (t0 + tb >= n) break;
+      float k[NB][8], v[NB], sk[NB], sq[NB];
+#pragma unroll
+      for (int j = 0; j < NB; ++j) {
+        const float *kp = &kq_s[stage][tb + j][0][r0], *qp = &kq_s[stage][tb + j][1][r0];
+        const float4 ka = *(const float4 *)kp, kb = *(const float4 *)(kp + 4), qa = *(const float4 *)qp, qb = *(const float4 *)(qp + 4);
+        k[j][0] = ka.x; k[j][1] = ka.y; k[j][2] = ka.z; k[j][3] = ka.w; k[j][4] = kb.x; k[j][5] = kb.y; k[j][6] = kb.z; k[j][7] = kb.w;
+        const float q[8] = {qa.x, qa.y, qa.z, qa.w, qb.x, qb.y, qb.z, qb.w};
+        v[j] = v_s[stage][tb + j][cl];
+        sk[j] = sq[j] = 0.0f;
+#pragma unroll
+        for (int r = 0; r < 8; ++r) {
+          sk[j] = __builtin_fmaf(S[r], k[j][r], sk[j]);
+          sq[j] = __builtin_fmaf(S[r], q[r], sq[j]);
+        }
       }
-      sk = column_sum<LPC>(sk);
-      sq = column_sum<LPC>(sq);
-      const float u = beta * (v_s[stage][t][cl] - g * sk);
 #pragma unroll
-      for (int r = 0; r < 8; ++r) S[r] = __builtin_fmaf(k[r], u, g * S[r]);
-      if (r0 == 0 && col < V && t0 + t < n) a.o[((size_t)((t0 + t) * a.batch + b) * s.heads + h) * V + col] = __builtin_fmaf(u, kq, g * sq);
+      for (int j = 0; j < NB; ++j) {
+        sk[j] = column_sum<LPC>(sk[j]);
+        sq[j] = column_sum<LPC>(sq[j]);
+      }
+      // Scalar loads and LDS reads count on one counter and scalar loads come back in any order, so a wait for LDS waits for
+      // them too: the next block's numbers are asked for here, behind this block's last LDS read.
+      __builtin_amdgcn_sched_barrier(0);
+      cf[(tb / NB + 1) & 1].load(coef + (size_t)min(t0 + tb + NB, w.padded - NB) * NCF);
+      __builtin_amdgcn_sched_barrier(0);
+      const Coefs &now = cf[(tb / NB) & 1];
+      float u[NB];
+#pragma unroll
+      for (int j = 0; j < NB; ++j) {
+        float e = __builtin_fmaf(-now.v[j][CF_GAMMA], sk[j], v[j]), o = now.v[j][CF_GAMMA] * sq[j];
+#pragma unroll
+        for (int d = 1; d <= j; ++d) {
+          e = __builtin_fmaf(-now.v[j][CF_KK + d - 1], u[j - d], e);
+          o = __builtin_fmaf(now.v[j][CF_KQ + d], u[j - d], o);
+        }
+        u[j] = now.v[j][CF_BETA] * e;
+        o = __builtin_fmaf(now.v[j][CF_KQ], u[j], o);
+        if (r0 == 0 && col < V && t0 + tb + j < n) a.o[((size_t)((t0 + tb + j) * a.batch + b) * s.heads + h) * V + col] = o;
+      }
+#pragma unroll
+      for (int r = 0; r < 8; ++r) S[r] *= now.v[NB - 1][CF_GAMMA];
+#pragma unroll
+      for (int j = 0; j < NB; ++j) {
+        const float y = u[j] * now.v[j][CF_END];
+#pragma unroll
+        for (int r = 0; r < 8; ++r) S[r] = __builtin_fmaf(k[j][r], y, S[r]);
+      }
     }
     if (t0 + CT < n) put(stage ^ 1);
     __syncthreads();
@@ -265,7 +384,13 @@ int kx_delta_launch(const KxDeltaArgs &a, hipStream_t st) {
     return KX_OK;
   }
   KX_REQUIRE(a.work, "delta rule: no scratch");
-  hipLaunchKernelGGL(delta_prep_k, dim3(a.batch * a.positions), dim3(256), 0, st, a);
+  const dim3 conv_grid(kx_cdiv(kx_delta_channels(s), 256), kx_cdiv(a.positions, CONV_TOKENS), a.batch);
+  if (s.taps == 2) hipLaunchKernelGGL(delta_conv_k<2>, conv_grid, dim3(256), 0, st, a);
+  else if (s.taps == 3) hipLaunchKernelGGL(delta_conv_k<3>, conv_grid, dim3(256), 0, st, a);
+  else if (s.taps == 4) hipLaunchKernelGGL(delta_conv_k<4>, conv_grid, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL(delta_conv_k<0>, conv_grid, dim3(256), 0, st, a);
+  KX_LAUNCH_CHECK();
+  hipLaunchKernelGGL(delta_unit_k, dim3(kx_cdiv(work_of(a).padded * s.kv_heads, 4), a.batch), dim3(256), 0, st, a);
   KX_LAUNCH_CHECK();
   if (s.taps > 1) {
     hipLaunchKernelGGL(delta_hist_k, dim3(kx_cdiv(kx_delta_channels(s), 256), a.batch), dim3(256), 0, st, a);

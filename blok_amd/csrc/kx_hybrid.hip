@@ -224,7 +224,7 @@ size_t HybridModel::layout(char *base) {
       w.dt_bias = vec(m + "dt_bias", d.heads, 0, -2.0f, 0.5f);
       w.o_norm = vec(m + "norm", d.vdim, 0, 1.0f, 0.02f);
       o_cols = std::max(o_cols, (size_t)out_cols);
-      work_floats = std::max(work_floats, kx_delta_work_floats(d));
+      work_floats = std::max(work_floats, kx_delta_work_floats(d, 1, step_tokens + max_batch * (KX_DELTA_BLOCK - 1)));  // a batch's sequences are padded to blocks each
       w.state_floats = (size_t)d.heads * d.dim * d.vdim;
       w.hist_floats = (size_t)(d.taps - 1) * C;
     }
@@ -265,7 +265,7 @@ size_t HybridModel::layout(char *base) {
   streams = (float *)at(T * S * W * 4);
   proj = (float *)at(T * proj_ld * 4);
   delta_o = (float *)at(T * o_cols * 4);
-  work = (float *)at(T * work_floats * 4);
+  work = (float *)at(work_floats * 4);
   part = (float *)at(part_floats * 4);
   rows = at(std::max(T, (size_t)logit_rows()) * row_ld * es);
   att = at(T * att_ld * es);

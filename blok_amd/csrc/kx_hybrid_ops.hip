@@ -91,7 +91,7 @@ extern "C" int kx_delta_create(const kx_delta_config *c, int32_t max_batch, int3
   d->max_batch = max_batch; d->max_positions = max_positions;
   d->state_bytes = (size_t)max_batch * s.heads * s.dim * s.vdim * 4;
   d->hist_bytes = (size_t)max_batch * (s.taps - 1) * kx_delta_channels(s) * 4;
-  const size_t total = d->state_bytes + 2 * d->hist_bytes + kx_delta_work_floats(s) * max_batch * max_positions * 4;
+  const size_t total = d->state_bytes + 2 * d->hist_bytes + kx_delta_work_floats(s, max_batch, max_positions) * 4;
   if (hipMalloc((void **)&d->mem, total) != hipSuccess || hipMemset(d->mem, 0, total) != hipSuccess) {
     kx_set_error("kx_delta_create: no device memory for %zu bytes", total);
     kx_delta_destroy(d);

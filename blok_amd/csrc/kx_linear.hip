@@ -31,83 +31,112 @@ __device__ __forceinline__ void put_glu(const KxLinArgs &a, int t, int col, floa
   u = fminf(fmaxf(u, -a.limit), a.limit);
   ((T *)a.mid)[(size_t)t * a.mid_ld + col] = Elem<T>::make(g * kx_sigmoidf(a.alpha * g) * (u + a.bias));
 }
-__device__ __forceinline__ void put_streams(const KxLinArgs &a, int t, int r, float y) {
-  float *x = a.streams + (size_t)t * a.n_streams * a.m.rows + r;
-  if (!a.mix) {
-    *x += y;
-    return;
+// EPI of the kernels: KX_LIN_F32, KX_LIN_GLU, or KX_LIN_STREAMS + number of streams (streams_any: up to KX_MAX_STREAMS)
+constexpr int STREAMS_ANY = KX_LIN_STREAMS + KX_MAX_STREAMS;
+__host__ __device__ constexpr int most_streams(int epi) { return epi > KX_LIN_STREAMS ? epi - KX_LIN_STREAMS : 1; }
+// The streams of one element of the residual row, read early and written late.  The small matrices come through the scalar
+// cache: every lane uses the same numbers and nothing writes them.
+typedef const __attribute__((address_space(4))) float *ScalarPtr;
+template <int EPI>
+struct Streams {
+  static constexpr int S = most_streams(EPI);
+  float old[S];
+  static __device__ __forceinline__ bool has(const KxLinArgs &a, int s) { return EPI != STREAMS_ANY || s < a.n_streams; }
+  __device__ __forceinline__ void load(const KxLinArgs &a, int t, int r) {
+    const float *x = a.streams + (size_t)t * a.n_streams * a.m.rows + r;
+#pragma unroll
+    for (int s = 0; s < S; ++s) old[s] = x[(size_t)(has(a, s) ? s : 0) * a.m.rows];
   }
-  float old[KX_MAX_STREAMS];
-#pragma unroll
-  for (int s = 0; s < KX_MAX_STREAMS; ++s)
-    if (s < a.n_streams) old[s] = x[(size_t)s * a.m.rows];
-#pragma unroll
-  for (int d = 0; d < KX_MAX_STREAMS; ++d)
-    if (d < a.n_streams) {
-      float v = a.outw[d] * y;
-#pragma unroll
-      for (int s = 0; s < KX_MAX_STREAMS; ++s)
-        if (s < a.n_streams) v = __builtin_fmaf(a.mix[s * a.n_streams + d], old[s], v);
-      x[(size_t)d * a.m.rows] = v;
+  __device__ __forceinline__ void store(const KxLinArgs &a, int t, int r, float y) const {
+    float *x = a.streams + (size_t)t * a.n_streams * a.m.rows + r;
+    if (!a.mix) {
+      *x = old[0] + y;
+      return;
     }
-}
+    const ScalarPtr mix = (ScalarPtr)a.mix, outw = (ScalarPtr)a.outw;
+    const int n = EPI == STREAMS_ANY ? a.n_streams : S;
+#pragma unroll
+    for (int d = 0; d < S; ++d) {
+      if (has(a, d)) {
+        float v = outw[d] * y;
+#pragma unroll
+        for (int s = 0; s < S; ++s)
+          if (has(a, s)) v = __builtin_fmaf(mix[s * n + d], old[s], v);
+        x[(size_t)d * a.m.rows] = v;
+      }
+    }
+  }
+};
 
 // matrix row of half i (0, 1) of unit k: a (gate, up) pair, or two consecutive rows
-__device__ __forceinline__ int unit_row(int epi, int k, int i) {
-  return epi == KX_LIN_GLU ? (k / KX_GLU_BLOCK) * (2 * KX_GLU_BLOCK) + (k % KX_GLU_BLOCK) + i * KX_GLU_BLOCK : 2 * k + i;
+template <int EPI>
+__device__ __forceinline__ int unit_row(int k, int i) {
+  return EPI == KX_LIN_GLU ? (k / KX_GLU_BLOCK) * (2 * KX_GLU_BLOCK) + (k % KX_GLU_BLOCK) + i * KX_GLU_BLOCK : 2 * k + i;
 }
 
 constexpr int GEMV_WAVES = 8, UP = 4;  // UP: pieces per row in flight
+__host__ __device__ __forceinline__ int gemv_row(int ld) { return (ld + 64 * UP * 8 - 1) / (64 * UP * 8) * (64 * UP * 8); }
 
-template <class T, int NT>
+template <class T, int NT, int EPI>
 __global__ void __launch_bounds__(GEMV_WAVES * 64) __attribute__((amdgpu_waves_per_eu(sizeof(T) == 2 ? 4 : 2)))
 lin_gemv_k(KxLinArgs a) {
   using E = Elem<T>;
   extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
   __shared__ float red[GEMV_WAVES][2 * NT];
-  T *xs = (T *)lds;                                            // [NT][ld]
-  float *u = (float *)(lds + (size_t)NT * a.m.ld * sizeof(T));  // row scratch
+  const int xl = gemv_row(a.m.ld);                          // a row in LDS, with zeros up to whole passes of the wave
+  T *xs = (T *)lds;                                         // [NT][xl]
+  float *u = (float *)(lds + (size_t)NT * xl * sizeof(T));  // row scratch
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int ld = a.m.ld, np = ld >> 3, nc = (np + 64 * UP - 1) / (64 * UP);
   const int units = (a.m.rows + 1) >> 1, nblk = (units + GEMV_WAVES - 1) / GEMV_WAVES;
   const T *w = (const T *)a.m.w;
-  typename E::Raw cur[2][UP], nxt[2][UP];
+  typename E::Raw bufA[2][UP], bufB[2][UP];
+  // Past the last block the first row is asked for once more, by every wave: the number of loads in flight has to be the
+  // same on every path, or the compiler waits for all of them.
   auto load = [&](typename E::Raw (&b)[2][UP], int blk, int c) {
-    const int k = min(blk * GEMV_WAVES + wave, units - 1);
+    const int k = blk < nblk ? min(blk * GEMV_WAVES + wave, units - 1) : 0;
+    if (blk >= nblk) c = 0;
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
-      const T *wr = w + (size_t)min(unit_row(a.epi, k, i), a.m.rows - 1) * ld;
+      const T *wr = w + (size_t)min(unit_row<EPI>(k, i), a.m.rows - 1) * ld;
 #pragma unroll
       for (int j = 0; j < UP; ++j) {
         const int p = (c * UP + j) * 64 + lane;
-        b[i][j] = p < np ? E::stream(wr + p * 8) : E::zero();
+        b[i][j] = E::stream(wr + min(p, np - 1) * 8);  // a lane past the row meets zeros
       }
     }
   };
   int blk = blockIdx.x, c = 0;
-  load(cur, blk, 0);
+  load(bufA, blk, 0);
 #pragma unroll
   for (int t = 0; t < NT; ++t)
-    if (t < a.tokens) kxr::build_row<T>(a.row, t, xs + (size_t)t * ld, ld, u);
+    if (t < a.tokens) {
+      for (int x = ld + threadIdx.x; x < xl; x += GEMV_WAVES * 64) xs[(size_t)t * xl + x] = E::make(0.0f);
+      kxr::build_row<T>(a.row, t, xs + (size_t)t * xl, ld, u);
+    }
   float acc[2 * NT];
 #pragma unroll
   for (int v = 0; v < 2 * NT; ++v) acc[v] = 0.0f;
-  while (blk < nblk) {
+  auto step = [&](typename E::Raw (&cur)[2][UP], typename E::Raw (&nxt)[2][UP]) {  // one chunk of columns of one unit per wave
     const bool last = c + 1 == nc;
     const int nblk_ = last ? blk + gridDim.x : blk, nc_ = last ? 0 : c + 1;
-    if (nblk_ < nblk) load(nxt, nblk_, nc_);
+    // lane i * NT + t < 2 NT finishes row i of the unit for token t; what it updates is asked for ahead of the next weights
+    const int unit = blk * GEMV_WAVES + wave, row = unit_row<EPI>(unit, lane / NT & 1), tok = NT > 1 ? lane % NT : 0;
+    const bool finish = EPI == KX_LIN_GLU ? lane < NT && tok < a.tokens && unit < units : lane < 2 * NT && row < a.m.rows && tok < a.tokens;
+    Streams<EPI> res;
+    if (EPI >= KX_LIN_STREAMS && last && finish) res.load(a, tok, row);
+    load(nxt, nblk_, nc_);
+    __builtin_amdgcn_sched_barrier(0);  // these loads are on their way before the last ones are waited for
 #pragma unroll
     for (int j = 0; j < UP; ++j) {
       const int p = (c * UP + j) * 64 + lane;
-      if ((c * UP + j) * 64 >= np) break;
-      const int q = min(p, np - 1);  // lanes past the row hold zero weights
       float wf[2][8];
       E::unpack(wf[0], cur[0][j]);
       E::unpack(wf[1], cur[1][j]);
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
         float xf[8];
-        E::unpack(xf, E::cached(xs + (size_t)(NT > 1 ? min(t, a.tokens - 1) : 0) * ld + q * 8));
+        E::unpack(xf, E::cached(xs + (size_t)(NT > 1 ? min(t, a.tokens - 1) : 0) * xl + p * 8));
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
           acc[t] = __builtin_fmaf(wf[0][e], xf[e], acc[t]);
@@ -121,28 +150,23 @@ lin_gemv_k(KxLinArgs a) {
 #pragma unroll
         for (int j = 0; j < kxw::reduce_out<2 * NT, 64>(); ++j) red[wave][kxw::reduce_index<2 * NT, 64>(lane, j)] = acc[j];
       asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // the wave reads its own sums back
-      const int k = blk * GEMV_WAVES + wave;
-      if (k < units) {
-        if (a.epi == KX_LIN_GLU) {
-          if (lane < a.tokens) put_glu<T>(a, lane, k, red[wave][lane], red[wave][NT + lane]);
-        } else if (lane < 2 * NT) {
-          const int i = lane / NT, t = lane % NT, r = 2 * k + i;
-          if (r < a.m.rows && t < a.tokens) {
-            if (a.epi == KX_LIN_F32) a.out[(size_t)t * a.out_ld + r] = red[wave][lane];
-            else put_streams(a, t, r, red[wave][lane]);
-          }
-        }
+      if (finish) {
+        if constexpr (EPI == KX_LIN_GLU) put_glu<T>(a, tok, unit, red[wave][lane], red[wave][NT + lane]);
+        else if constexpr (EPI == KX_LIN_F32) a.out[(size_t)tok * a.out_ld + row] = red[wave][lane];
+        else res.store(a, tok, row, red[wave][lane]);
       }
       asm volatile("" ::: "memory");
 #pragma unroll
       for (int v = 0; v < 2 * NT; ++v) acc[v] = 0.0f;
     }
-#pragma unroll
-    for (int i = 0; i < 2; ++i)
-#pragma unroll
-      for (int j = 0; j < UP; ++j) cur[i][j] = nxt[i][j];
     blk = nblk_;
     c = nc_;
+  };
+  for (;;) {
+    step(bufA, bufB);
+    if (blk >= nblk) break;
+    step(bufB, bufA);
+    if (blk >= nblk) break;
   }
 }
 
@@ -154,7 +178,7 @@ __global__ void __launch_bounds__(256) row_k(KxRowArgs a, T *out, int ld) {
 
 // ---- bf16 GEMM ----
 // 4 waves as 2 x 2: wave (wm, wn) owns MI blocks of 32 tokens and 64 rows (two blocks of 32: with GLU rows, gate and up).
-template <int MI>
+template <int MI, int EPI>
 __global__ void __launch_bounds__(256, 2) lin_gemm_k(KxLinArgs a, const uint16_t *__restrict__ x, int x_ld) {
   constexpr int BM = MI * 64, BN = 128, ROWS = BM + BN, STAGE = ROWS * 128, CPW = ROWS / 32;
   extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
@@ -207,28 +231,41 @@ __global__ void __launch_bounds__(256, 2) lin_gemm_k(KxLinArgs a, const uint16_t
   }
   // D[i][j]: j = lane % 32 (row of the matrix), i = 8 (v / 4) + 4 (lane / 32) + v % 4 (token)
   const int rg = n0 + wn * 64 + lr;
+  auto token = [&](int i, int v) { return m0 + (wm * MI + i) * 32 + 8 * (v >> 2) + 4 * h + (v & 3); };
 #pragma unroll
-  for (int i = 0; i < MI; ++i)
+  for (int i = 0; i < MI; ++i) {
+    if constexpr (EPI == KX_LIN_GLU) {
 #pragma unroll
-    for (int v = 0; v < 16; ++v) {
-      const int t = m0 + (wm * MI + i) * 32 + 8 * (v >> 2) + 4 * h + (v & 3);
-      if (t >= a.tokens) continue;
-      if (a.epi == KX_LIN_GLU) {
-        if (rg < a.m.rows) put_glu<uint16_t>(a, t, (n0 + wn * 64) / 2 + lr, acc[i][0][v], acc[i][1][v]);
-      } else {
+      for (int v = 0; v < 16; ++v)
+        if (token(i, v) < a.tokens && rg < a.m.rows) put_glu<uint16_t>(a, token(i, v), (n0 + wn * 64) / 2 + lr, acc[i][0][v], acc[i][1][v]);
+    } else {
 #pragma unroll
-        for (int j = 0; j < 2; ++j) {
-          const int r = rg + 32 * j;
-          if (r >= a.m.rows) continue;
-          if (a.epi == KX_LIN_F32) a.out[(size_t)t * a.out_ld + r] = acc[i][j][v];
-          else put_streams(a, t, r, acc[i][j][v]);
+      for (int j = 0; j < 2; ++j) {
+        const int r = rg + 32 * j;
+        if constexpr (EPI == KX_LIN_F32) {
+#pragma unroll
+          for (int v = 0; v < 16; ++v)
+            if (token(i, v) < a.tokens && r < a.m.rows) a.out[(size_t)token(i, v) * a.out_ld + r] = acc[i][j][v];
+        } else {
+          constexpr int G = most_streams(EPI) > 2 ? 4 : 16;  // elements read before the first is written
+#pragma unroll
+          for (int v0 = 0; v0 < 16; v0 += G) {
+            Streams<EPI> res[G];
+#pragma unroll
+            for (int v = 0; v < G; ++v) res[v].load(a, min(token(i, v0 + v), a.tokens - 1), min(r, a.m.rows - 1));
+#pragma unroll
+            for (int v = 0; v < G; ++v)
+              if (token(i, v0 + v) < a.tokens && r < a.m.rows) res[v].store(a, token(i, v0 + v), r, acc[i][j][v0 + v]);
+          }
         }
       }
     }
+  }
 }
 
 // ---- f32 GEMM: 64 tokens x 64 rows, a thread owns 4 x 4; its rows are r, r + 16, ..., so that (gate, up) pairs, 32
 // rows apart, meet in one thread ----
+template <int EPI>
 __global__ void __launch_bounds__(256) lin_gemm_f32_k(KxLinArgs a, const float *__restrict__ x, int x_ld) {
   constexpr int BK = 16, STR = 68;
   __shared__ float xs[BK][STR], ws[BK][STR];
@@ -266,42 +303,44 @@ __global__ void __launch_bounds__(256) lin_gemm_f32_k(KxLinArgs a, const float *
     for (int j = 0; j < 4; ++j) {
       const int r = n0 + tx + 16 * j;
       if (r >= a.m.rows) continue;
-      if (a.epi == KX_LIN_F32) a.out[(size_t)t * a.out_ld + r] = acc[i][j];
-      else if (a.epi == KX_LIN_STREAMS) put_streams(a, t, r, acc[i][j]);
-      else if (j < 2) put_glu<float>(a, t, n0 / 2 + tx + 16 * j, acc[i][j], acc[i][j + 2]);
+      if constexpr (EPI == KX_LIN_F32) {
+        a.out[(size_t)t * a.out_ld + r] = acc[i][j];
+      } else if constexpr (EPI == KX_LIN_GLU) {
+        if (j < 2) put_glu<float>(a, t, n0 / 2 + tx + 16 * j, acc[i][j], acc[i][(j + 2) & 3]);
+      } else {
+        Streams<EPI> res;
+        res.load(a, t, r);
+        res.store(a, t, r, acc[i][j]);
+      }
     }
   }
 }
 
 constexpr size_t GEMV_LDS = 150 * 1024;
 
-template <class T, int NT>
-int gemv(const KxLinArgs &a, size_t lds, hipStream_t st) {
+template <class T, int NT, int EPI>
+int gemv_nt(const KxLinArgs &a, size_t lds, hipStream_t st) {
   static std::atomic<bool> attr{false};  // setting it twice from two threads is harmless
   if (!attr) {
-    KX_HIP(hipFuncSetAttribute((const void *)lin_gemv_k<T, NT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)GEMV_LDS));
+    KX_HIP(hipFuncSetAttribute((const void *)lin_gemv_k<T, NT, EPI>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)GEMV_LDS));
     attr = true;
   }
   const int nblk = kx_cdiv((a.m.rows + 1) / 2, GEMV_WAVES);
-  hipLaunchKernelGGL((lin_gemv_k<T, NT>), dim3(std::min(nblk, 2 * std::max(1, kx_device_cus()))), dim3(GEMV_WAVES * 64), lds, st, a);
+  hipLaunchKernelGGL((lin_gemv_k<T, NT, EPI>), dim3(std::min(nblk, 2 * std::max(1, kx_device_cus()))), dim3(GEMV_WAVES * 64), lds, st, a);
   KX_LAUNCH_CHECK();
   return KX_OK;
 }
 
-template <class T>
-int linear(const KxLinArgs &a, void *row_buf, hipStream_t st) {
-  KX_REQUIRE(a.m.w && a.m.rows > 0 && a.m.cols > 0 && a.m.ld >= a.m.cols && a.m.ld % KX_LD == 0, "kx_linear: matrix of %d x %d (%d)", a.m.rows, a.m.cols, a.m.ld);
-  KX_REQUIRE(a.tokens > 0 && a.row.cols == a.m.cols, "kx_linear: tokens=%d, rows of %d for %d columns", a.tokens, a.row.cols, a.m.cols);
-  KX_REQUIRE(a.epi != KX_LIN_GLU || a.m.rows % (2 * KX_GLU_BLOCK) == 0, "kx_linear: %d rows are no (gate, up) blocks", a.m.rows);
-  KX_REQUIRE(a.n_streams >= 1 && a.n_streams <= KX_MAX_STREAMS && (a.mix || a.n_streams == 1), "kx_linear: %d streams", a.n_streams);
+template <class T, int EPI>
+int linear_epi(const KxLinArgs &a, void *row_buf, hipStream_t st) {
   const size_t scratch = (size_t)kx_row_scratch(a.row) * 4;
   if (a.tokens <= KX_GEMV_TOKENS) {
     const int nt = a.tokens > 2 ? 4 : a.tokens;
-    const size_t lds = (size_t)nt * a.m.ld * sizeof(T) + scratch;
+    const size_t lds = (size_t)nt * gemv_row(a.m.ld) * sizeof(T) + scratch;
     if (lds <= GEMV_LDS) {
-      if (nt == 1) return gemv<T, 1>(a, lds, st);
-      if (nt == 2) return gemv<T, 2>(a, lds, st);
-      return gemv<T, 4>(a, lds, st);
+      if (nt == 1) return gemv_nt<T, 1, EPI>(a, lds, st);
+      if (nt == 2) return gemv_nt<T, 2, EPI>(a, lds, st);
+      return gemv_nt<T, 4, EPI>(a, lds, st);
     }
   }
   const T *x = (const T *)a.row.x;
@@ -320,19 +359,50 @@ int linear(const KxLinArgs &a, void *row_buf, hipStream_t st) {
   }
   KX_REQUIRE(a.row.kind != KX_ROW_PLAIN || !a.row.rows_map, "kx_linear: mapped rows have to be built");
   KX_REQUIRE(x && x_ld >= a.m.ld, "kx_linear: activation rows of %d, the matrix has %d", x_ld, a.m.ld);
-  if constexpr (sizeof(T) == 4) {
-    hipLaunchKernelGGL(lin_gemm_f32_k, dim3(kx_cdiv(a.m.rows, 64), kx_cdiv(a.tokens, 64)), dim3(256), 0, st, a, x, x_ld);
+  if constexpr (sizeof(T) == 2 && EPI == STREAMS_ANY) {  // more streams than the matrix-core kernel is built for: a few tokens at a time
+    KX_REQUIRE(gemv_row(a.m.ld) * sizeof(T) <= GEMV_LDS, "kx_linear: rows of %d columns with %d streams do not fit a workgroup", a.m.ld, a.n_streams);
+    const int most = (size_t)4 * gemv_row(a.m.ld) * sizeof(T) <= GEMV_LDS ? 4 : 1;
+    for (int t = 0; t < a.tokens; t += most) {
+      KxLinArgs b = a;
+      b.row = KxRowArgs();
+      b.row.cols = a.row.cols; b.row.x = x + (size_t)t * x_ld; b.row.x_ld = x_ld;
+      b.tokens = std::min(most, a.tokens - t);
+      b.streams = a.streams + (size_t)t * a.n_streams * a.m.rows;
+      const size_t lds = (size_t)most * gemv_row(a.m.ld) * sizeof(T);
+      int rc = most == 4 ? gemv_nt<T, 4, EPI>(b, lds, st) : gemv_nt<T, 1, EPI>(b, lds, st);
+      if (rc) return rc;
+    }
+    return KX_OK;
+  } else if constexpr (sizeof(T) == 4) {
+    hipLaunchKernelGGL((lin_gemm_f32_k<EPI>), dim3(kx_cdiv(a.m.rows, 64), kx_cdiv(a.tokens, 64)), dim3(256), 0, st, a, x, x_ld);
   } else {
     static std::atomic<bool> attr{false};
     if (!attr) {
-      KX_HIP(hipFuncSetAttribute((const void *)lin_gemm_k<2>, hipFuncAttributeMaxDynamicSharedMemorySize, 64 * 1024));
+      KX_HIP(hipFuncSetAttribute((const void *)lin_gemm_k<2, EPI>, hipFuncAttributeMaxDynamicSharedMemorySize, 64 * 1024));
       attr = true;
     }
-    if (a.tokens > 64) hipLaunchKernelGGL(lin_gemm_k<2>, dim3(kx_cdiv(a.m.rows, 128), kx_cdiv(a.tokens, 128)), dim3(256), 2 * 256 * 128, st, a, x, x_ld);
-    else hipLaunchKernelGGL(lin_gemm_k<1>, dim3(kx_cdiv(a.m.rows, 128), 1), dim3(256), 2 * 192 * 128, st, a, x, x_ld);
+    if (a.tokens > 64) hipLaunchKernelGGL((lin_gemm_k<2, EPI>), dim3(kx_cdiv(a.m.rows, 128), kx_cdiv(a.tokens, 128)), dim3(256), 2 * 256 * 128, st, a, x, x_ld);
+    else hipLaunchKernelGGL((lin_gemm_k<1, EPI>), dim3(kx_cdiv(a.m.rows, 128), 1), dim3(256), 2 * 192 * 128, st, a, x, x_ld);
   }
   KX_LAUNCH_CHECK();
   return KX_OK;
+}
+
+template <class T>
+int linear(const KxLinArgs &a, void *row_buf, hipStream_t st) {
+  KX_REQUIRE(a.m.w && a.m.rows > 0 && a.m.cols > 0 && a.m.ld >= a.m.cols && a.m.ld % KX_LD == 0, "kx_linear: matrix of %d x %d (%d)", a.m.rows, a.m.cols, a.m.ld);
+  KX_REQUIRE(a.tokens > 0 && a.row.cols == a.m.cols, "kx_linear: tokens=%d, rows of %d for %d columns", a.tokens, a.row.cols, a.m.cols);
+  KX_REQUIRE(a.epi != KX_LIN_GLU || a.m.rows % (2 * KX_GLU_BLOCK) == 0, "kx_linear: %d rows are no (gate, up) blocks", a.m.rows);
+  KX_REQUIRE(a.n_streams >= 1 && a.n_streams <= KX_MAX_STREAMS && (a.mix || a.n_streams == 1), "kx_linear: %d streams", a.n_streams);
+  if (a.epi == KX_LIN_F32) return linear_epi<T, KX_LIN_F32>(a, row_buf, st);
+  if (a.epi == KX_LIN_GLU) return linear_epi<T, KX_LIN_GLU>(a, row_buf, st);
+  if constexpr (sizeof(T) == 2) {
+    if (a.n_streams == 1) return linear_epi<T, KX_LIN_STREAMS + 1>(a, row_buf, st);
+    if (a.n_streams == 2) return linear_epi<T, KX_LIN_STREAMS + 2>(a, row_buf, st);
+    if (a.n_streams == 3) return linear_epi<T, KX_LIN_STREAMS + 3>(a, row_buf, st);
+    if (a.n_streams == 4) return linear_epi<T, KX_LIN_STREAMS + 4>(a, row_buf, st);
+  }
+  return linear_epi<T, STREAMS_ANY>(a, row_buf, st);
 }
 
 }  // namespace

@@ -22,7 +22,6 @@ template <> struct Elem<uint16_t> {
   static __device__ __forceinline__ uint16_t make(float v) { return kx_bf16_rne(v); }
   // eight elements of a weight stream, as they come
   struct Raw { u32x4 a; };
-  static __device__ __forceinline__ Raw zero() { return Raw{u32x4{0, 0, 0, 0}}; }
   static __device__ __forceinline__ Raw stream(const uint16_t *p) { return Raw{__builtin_nontemporal_load((const u32x4 *)p)}; }
   static __device__ __forceinline__ Raw cached(const uint16_t *p) { return Raw{*(const u32x4 *)p}; }
   static __device__ __forceinline__ void unpack(float (&f)[8], const Raw &r) {
@@ -37,7 +36,6 @@ template <> struct Elem<float> {
   static __device__ __forceinline__ float load(const float *p) { return *p; }
   static __device__ __forceinline__ float make(float v) { return v; }
   struct Raw { u32x4 a, b; };
-  static __device__ __forceinline__ Raw zero() { return Raw{u32x4{0, 0, 0, 0}, u32x4{0, 0, 0, 0}}; }
   static __device__ __forceinline__ Raw stream(const float *p) {
     return Raw{__builtin_nontemporal_load((const u32x4 *)p), __builtin_nontemporal_load((const u32x4 *)(p + 4))};
   }

@@ -235,26 +235,37 @@ __global__ void __launch_bounds__(PART_THREADS) win_partial_k(KxWindowArgs a, in
   }
 }
 
-// the parts of one head of one token merged, with the sink, times sigmoid(gate)
+// the parts of one head of one token merged, with the sink, times sigmoid(gate); one wave finds the parts' weights
+constexpr int MERGE_THREADS = 128;
 template <class T>
-__global__ void __launch_bounds__(128) win_merge_k(KxWindowArgs a, int tok0, int parts, const float *po, const float *pm, const float *pz) {
+__global__ void __launch_bounds__(MERGE_THREADS) win_merge_k(KxWindowArgs a, int tok0, int parts, const float *po, const float *pm, const float *pz) {
+  extern __shared__ float weight[];  // [parts]
   const KxWindowSpec &s = a.s;
-  const int h = blockIdx.x, tok = tok0 + blockIdx.y;
+  const int h = blockIdx.x, tok = tok0 + blockIdx.y, tid = threadIdx.x;
   const size_t row = (size_t)blockIdx.y * parts;
-  float m = s.sink ? 0.0f : NEG_INF;
-  for (int k = 0; k < parts; ++k) m = fmaxf(m, pm[(row + k) * s.heads + h]);
-  float z = s.sink ? kx_expf(-m) : 0.0f;
-  for (int k = 0; k < parts; ++k) z = __builtin_fmaf(pz[(row + k) * s.heads + h], kx_expf(pm[(row + k) * s.heads + h] - m), z);
-  T *out = (T *)a.out + (size_t)tok * a.out_ld + h * s.vdim;
-  for (int d = threadIdx.x; d < s.vdim; d += 128) {
-    float v = 0.0f;
-    for (int k = 0; k < parts; ++k) {
+  if (tid < 64) {
+    float m = s.sink ? 0.0f : NEG_INF, z = 0.0f;
+    for (int k = tid; k < parts; k += 64) m = fmaxf(m, pm[(row + k) * s.heads + h]);
+    m = kxw::wave_max_f32(m);
+    for (int k = tid; k < parts; k += 64) {
       const float w = kx_expf(pm[(row + k) * s.heads + h] - m);
-      if (w > 0.0f) v = __builtin_fmaf(po[((row + k) * s.heads + h) * a.c.vp + d], w, v);
+      weight[k] = w;
+      z = __builtin_fmaf(pz[(row + k) * s.heads + h], w, z);
     }
-    v /= z;
-    if (a.g_off >= 0) v *= kx_sigmoidf(a.proj[(size_t)tok * a.proj_ld + a.g_off + h * s.vdim + d]);
-    out[d] = Elem<T>::make(v);
+    const float inv = 1.0f / (kxr::wave_sum(z) + (s.sink ? kx_expf(-m) : 0.0f));
+    for (int k = tid; k < parts; k += 64) weight[k] *= inv;
+  }
+  __syncthreads();
+  T *out = (T *)a.out + (size_t)tok * a.out_ld + h * s.vdim;
+  for (int d = tid; d < s.vdim; d += MERGE_THREADS) {
+    const float gate = a.g_off >= 0 ? kx_sigmoidf(a.proj[(size_t)tok * a.proj_ld + a.g_off + h * s.vdim + d]) : 1.0f;
+    float v = 0.0f;
+#pragma unroll 8
+    for (int k = 0; k < parts; ++k) {  // a part without keys has not written its sums
+      const float x = po[((row + k) * s.heads + h) * a.c.vp + d];
+      v = weight[k] > 0.0f ? __builtin_fmaf(x, weight[k], v) : v;
+    }
+    out[d] = Elem<T>::make(v * gate);
   }
 }
 
@@ -263,8 +274,11 @@ __global__ void __launch_bounds__(128) win_merge_k(KxWindowArgs a, int tok0, int
 // denominator are one value per lane, and the weights go from the first product's result into the second product's
 // operand without leaving the registers.  The result layout gives lane (q, h) the keys 8 (v / 4) + 4 h + v % 4 of a tile of
 // 32; the operand layout wants 8 keys in a row per lane, so within 16 keys the V^T tile stores keys 0-3, 8-11 for
-// h = 0 and 4-7, 12-15 for h = 1.
+// h = 0 and 4-7, 12-15 for h = 1.  The 8-key pieces of a V^T row are xor-swizzled by the row, which spreads the
+// transposing writes over the banks.  The next tile's rows are on their way to registers while a tile is multiplied;
+// scores are in units of log 2, so that a weight is one exp2.
 constexpr int FQ = 128, FK = 64;
+__device__ __forceinline__ int vt_piece(int d, int piece) { return (piece ^ (d >> 1) ^ (d >> 4)) & 7; }
 
 template <int ND, int NV>  // 32-column blocks of a key and of a value
 __global__ void __launch_bounds__(256) win_flash_k(KxWindowArgs a) {
@@ -296,40 +310,69 @@ __global__ void __launch_bounds__(256) win_flash_k(KxWindowArgs a) {
 #pragma unroll
     for (int v = 0; v < 16; ++v) o[j][v] = 0.0f;
   float m = s.sink ? 0.0f : NEG_INF, z = s.sink && hh == 0 ? 1.0f : 0.0f;  // z: this lane's half of the keys
+  const float scale2 = s.scale * 1.44269504088896341f;
 
   // tiles: the blocks the last query sees, then the positions from the first query's window on
   const int tb = (seen_blocks(p_last, s.size, s.pool) + FK - 1) / FK;
-  const int j0 = window_lo(p_first, s.size) & ~(FK - 1), tw = (p_last - j0) / FK + 1;
-  for (int t = 0; t < tb + tw; ++t) {
+  const int j0 = window_lo(p_first, s.size) & ~(FK - 1), tiles = tb + (p_last - j0) / FK + 1;
+  // what all and what any of this wave's queries see
+  const int q0 = __builtin_amdgcn_readfirstlane(a.pos + min(i0 + wave * 32, a.positions - 1));
+  const int q1 = __builtin_amdgcn_readfirstlane(a.pos + min(i0 + wave * 32 + 31, a.positions - 1));
+  const int nb0 = seen_blocks(q0, s.size, s.pool), nb1 = seen_blocks(q1, s.size, s.pool), lo0 = window_lo(q0, s.size), lo1 = window_lo(q1, s.size);
+  auto first_key = [&](int t) { return t < tb ? t * FK : j0 + (t - tb) * FK; };
+  constexpr int VT = (FK / 8) * NV * 16, VN = (VT + 255) / 256;  // V is taken by 8 keys x 2 columns
+  uint4 kreg[ND];
+  uint32_t vreg[VN][8];
+  // Rows of a tile: a window tile starts at a multiple of FK and the ring's length is one, so it does not wrap inside; past the
+  // last block there is nothing to read.  What is read beyond a row's columns or the keys a query sees meets zeros.
+  auto fetch = [&](int t) {
     const bool pooled = t < tb;
-    const int k0 = pooled ? t * FK : j0 + (t - tb) * FK;  // first block or position of the tile
-    const int klim = pooled ? c.blocks : p_last + 1;      // rows from here on are not read
-    __syncthreads();  // the tile before has been multiplied
-    // a row of the cache: a window tile starts at a multiple of FK and the ring's length is one, so it does not wrap inside
+    const int k0 = first_key(t), last = pooled ? c.blocks - 1 - k0 : FK - 1;
     const uint16_t *kr = pooled ? pkc + (size_t)k0 * c.dp : kc + (size_t)(k0 % c.cap) * c.dp;
     const uint16_t *vr = pooled ? pvc + (size_t)k0 * c.vp : vc + (size_t)(k0 % c.cap) * c.vp;
-    for (int x = tid; x < FK * ND * 4; x += 256) {
-      const int r = x / (ND * 4), d = (x - r * (ND * 4)) * 8;
-      uint4 w = make_uint4(0, 0, 0, 0);
-      if (k0 + r < klim && d < c.dp) w = *(const uint4 *)(kr + (size_t)r * c.dp + d);
-      *(uint4 *)(ks + r * KSTR + d) = w;
-    }
-    for (int x = tid; x < (FK / 8) * NV * 16; x += 256) {  // 8 keys x 2 value columns
-      const int oct = x / (NV * 16), d = (x - oct * (NV * 16)) * 2;
-      uint32_t w[8];
 #pragma unroll
-      for (int y = 0; y < 8; ++y) {
-        w[y] = 0;
-        if (k0 + oct * 8 + y < klim && d < c.vp) w[y] = *(const uint32_t *)(vr + (size_t)(oct * 8 + y) * c.vp + d);
-      }
-      const int at = (oct >> 1) * 16 + (oct & 1) * 4;  // keys 0-3 of the octet here, 4-7 eight places further
+    for (int y = 0; y < ND; ++y) {
+      const int x = y * 256 + tid, r = x / (ND * 4), d = (x - r * (ND * 4)) * 8;
+      kreg[y] = *(const uint4 *)(kr + (size_t)min(r, last) * c.dp + min(d, c.dp - 8));
+    }
 #pragma unroll
-      for (int y = 0; y < 2; ++y) {
-        *(u32x2 *)(vt + d * VSTR + at + y * 8) = u32x2{(w[4 * y] & 0xffffu) | (w[4 * y + 1] << 16), (w[4 * y + 2] & 0xffffu) | (w[4 * y + 3] << 16)};
-        *(u32x2 *)(vt + (d + 1) * VSTR + at + y * 8) = u32x2{(w[4 * y] >> 16) | (w[4 * y + 1] & 0xffff0000u), (w[4 * y + 2] >> 16) | (w[4 * y + 3] & 0xffff0000u)};
+    for (int y = 0; y < VN; ++y) {
+      const int x = min(y * 256 + tid, VT - 1), oct = x / (NV * 16), d = min((x - oct * (NV * 16)) * 2, c.vp - 2);
+#pragma unroll
+      for (int r = 0; r < 8; ++r) vreg[y][r] = *(const uint32_t *)(vr + (size_t)min(oct * 8 + r, last) * c.vp + d);
+    }
+  };
+  auto put = [&]() {
+#pragma unroll
+    for (int y = 0; y < ND; ++y) {
+      const int x = y * 256 + tid, r = x / (ND * 4), d = (x - r * (ND * 4)) * 8;
+      *(uint4 *)(ks + r * KSTR + d) = kreg[y];
+    }
+#pragma unroll
+    for (int y = 0; y < VN; ++y) {
+      const int x = y * 256 + tid, oct = x / (NV * 16), d = (x - oct * (NV * 16)) * 2;
+      if (x >= VT) continue;
+      const uint32_t *w = vreg[y];
+#pragma unroll
+      for (int half = 0; half < 2; ++half) {  // keys 0-3 of the octet, keys 4-7
+        const int at = vt_piece(d, (oct >> 1) * 2 + half) * 8 + (oct & 1) * 4;
+        const uint32_t *k4 = w + 4 * half;
+        *(u32x2 *)(vt + d * VSTR + at) = u32x2{(k4[0] & 0xffffu) | (k4[1] << 16), (k4[2] & 0xffffu) | (k4[3] << 16)};
+        *(u32x2 *)(vt + (d + 1) * VSTR + at) = u32x2{(k4[0] >> 16) | (k4[1] & 0xffff0000u), (k4[2] >> 16) | (k4[3] & 0xffff0000u)};
       }
     }
+  };
+  fetch(0);
+  for (int t = 0; t < tiles; ++t) {
+    const bool pooled = t < tb;
+    const int k0 = first_key(t);
+    __syncthreads();  // the tile before has been multiplied
+    put();
     __syncthreads();
+    if (t + 1 < tiles) fetch(t + 1);
+    const bool none = pooled ? k0 >= nb1 : k0 > q1 || k0 + FK - 1 < lo0;
+    const bool all = pooled ? k0 + FK <= nb0 : k0 >= lo1 && k0 + FK - 1 <= q0;
+    if (none) continue;
     f32x16 sc[2];
 #pragma unroll
     for (int kt = 0; kt < 2; ++kt) {
@@ -346,26 +389,30 @@ __global__ void __launch_bounds__(256) win_flash_k(KxWindowArgs a) {
     for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
       for (int v = 0; v < 16; ++v) {
-        const int e = k0 + kt * 32 + 8 * (v >> 2) + 4 * hh + (v & 3);
-        const bool see = pooled ? e < nb : e >= lo && e <= p;
-        sc[kt][v] = see ? sc[kt][v] * s.scale : NEG_INF;
+        sc[kt][v] *= scale2;
+        if (!all) {
+          const int e = k0 + kt * 32 + 8 * (v >> 2) + 4 * hh + (v & 3);
+          const bool see = pooled ? e < nb : e >= lo && e <= p;
+          sc[kt][v] = see ? sc[kt][v] : NEG_INF;
+        }
         tm = fmaxf(tm, sc[kt][v]);
       }
     tm = fmaxf(tm, __shfl_xor(tm, 32));
-    const float m1 = fmaxf(m, tm);
-    const float mm = m1 == NEG_INF ? 0.0f : m1;  // nothing seen so far
-    const float al = kx_expf(m - mm);
-    m = m1;
-    z *= al;
+    if (__any(tm > m)) {
+      const float m1 = fmaxf(m, tm), al = m == NEG_INF ? 0.0f : __builtin_amdgcn_exp2f(m - m1);
+      m = m1;
+      z *= al;
 #pragma unroll
-    for (int j = 0; j < NV; ++j)
+      for (int j = 0; j < NV; ++j)
 #pragma unroll
-      for (int v = 0; v < 16; ++v) o[j][v] *= al;
+        for (int v = 0; v < 16; ++v) o[j][v] *= al;
+    }
+    const float mm = m == NEG_INF ? 0.0f : m;  // nothing seen so far
 #pragma unroll
     for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
       for (int v = 0; v < 16; ++v) {
-        sc[kt][v] = __expf(sc[kt][v] - mm);
+        sc[kt][v] = __builtin_amdgcn_exp2f(sc[kt][v] - mm);
         z += sc[kt][v];
       }
 #pragma unroll
@@ -381,7 +428,8 @@ __global__ void __launch_bounds__(256) win_flash_k(KxWindowArgs a) {
       const bf16x8 pf = __builtin_bit_cast(bf16x8, make_uint4(pw[0], pw[1], pw[2], pw[3]));
 #pragma unroll
       for (int j = 0; j < NV; ++j) {
-        const bf16x8 vf = *(const bf16x8 *)(vt + (j * 32 + lq) * VSTR + ss * 16 + hh * 8);
+        const int d = j * 32 + lq;
+        const bf16x8 vf = *(const bf16x8 *)(vt + d * VSTR + vt_piece(d, ss * 2 + hh) * 8);
         o[j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, pf, o[j], 0, 0, 0);
       }
     }
@@ -473,7 +521,7 @@ int attention(const KxWindowArgs &a, hipStream_t st) {
     if (fused) hipLaunchKernelGGL((win_partial_k<T, true>), grid, dim3(PART_THREADS), lds, st, a, t0, ch, po, pm, pz);
     else hipLaunchKernelGGL((win_partial_k<T, false>), grid, dim3(PART_THREADS), lds, st, a, t0, ch, po, pm, pz);
     KX_LAUNCH_CHECK();
-    hipLaunchKernelGGL((win_merge_k<T>), dim3(s.heads, n), dim3(128), 0, st, a, t0, parts, po, pm, pz);
+    hipLaunchKernelGGL((win_merge_k<T>), dim3(s.heads, n), dim3(MERGE_THREADS), (size_t)parts * 4, st, a, t0, parts, po, pm, pz);
     KX_LAUNCH_CHECK();
   }
   return KX_OK;
