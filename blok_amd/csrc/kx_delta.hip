@@ -14,7 +14,7 @@
 //   S  <- D(4) S + sum_i D(i, 4) k_i u_i^T,
 // which is the recurrence written out for four tokens.  The numbers that do not depend on the column -- per token D(j),
 // beta, D(j, 4), D(j - d, j) (k_{j-d} . k_j) for d = 1..3 and D(j - d, j) (k_{j-d} . q_j) for d = 0..3 -- are made
-// once per head by delta_unit_k and come to the scan through scalar loads.
+// once per head by delta_unit_k.
 #include <algorithm>
 #include <atomic>
 #include "kx_common.h"
@@ -22,6 +22,8 @@
 #include "kx_delta.h"
 
 namespace {
+
+typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 constexpr int SC = 32;  // columns per workgroup of delta_step_k
 
@@ -249,100 +251,114 @@ __device__ __forceinline__ float column_sum(float v) {  // over the LPC lanes of
   return v;
 }
 
-// A block's numbers, through the scalar cache: they are the same for the whole workgroup and this kernel does not write them.
-typedef const __attribute__((address_space(4))) float *ScalarPtr;
+// A block's numbers, one per lane as they are loaded, in scalar registers as they are used: they are the same for the whole
+// workgroup.  (Scalar loads would come from the memory side of the caches, 1-2 us away, once per block.)
 struct Coefs {
   float v[NB][NCF];
-  __device__ __forceinline__ void load(const float *p) {
-    const ScalarPtr q = (ScalarPtr)p;
+  __device__ __forceinline__ void from_lanes(float x) {
 #pragma unroll
     for (int j = 0; j < NB; ++j)
 #pragma unroll
-      for (int x = 0; x < NCF; ++x) v[j][x] = q[j * NCF + x];
+      for (int y = 0; y < NCF; ++y) v[j][y] = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, x), j * NCF + y));
   }
 };
+static_assert(NB * NCF <= 64, "a block's numbers are one wave load");
 
 template <int LPC>  // lanes per column, 8 rows of the state each
 __global__ void __launch_bounds__(256) delta_scan_k(KxDeltaArgs a) {
   constexpr int DP = LPC * 8, COLS = 256 / LPC, CT = LPC >= 16 ? 16 : 32;  // CT: tokens per staged block
   __shared__ __attribute__((aligned(16))) float kq_s[2][CT][2][DP];
-  __shared__ float v_s[2][CT][COLS];
+  __shared__ float v_s[2][CT][COLS], o_s[2][CT][COLS];
   const KxDeltaSpec &s = a.s;
   const int D = s.dim, V = s.vdim, tid = threadIdx.x;
   const int h = blockIdx.y, b = blockIdx.z, c0 = blockIdx.x * COLS, kvh = h / (s.heads / s.kv_heads), nq = s.kv_heads * D;
-  const int C = kx_delta_channels(s), r0 = (tid % LPC) * 8, cl = tid / LPC, col = c0 + cl, n = a.positions;
+  const int C = kx_delta_channels(s), l4 = (tid % LPC) * 4, cl = tid / LPC, col = c0 + cl, n = a.positions;
   const Work w = work_of(a);
   const float *coef = w.coef + ((size_t)b * s.heads + h) * w.padded * NCF;
   float *st = a.state + ((size_t)b * s.heads + h) * D * V;
+  auto row = [&](int r) { return (r < 4 ? 0 : DP / 2 - 4) + l4 + r; };  // two runs of four rows: neighbouring lanes read neighbouring words
   float S[8];
 #pragma unroll
-  for (int r = 0; r < 8; ++r) S[r] = r0 + r < D && col < V ? st[(size_t)(r0 + r) * V + col] : 0.0f;
+  for (int r = 0; r < 8; ++r) S[r] = row(r) < D && col < V ? st[(size_t)row(r) * V + col] : 0.0f;
   // A stage of tokens goes through registers into one of two LDS stages while the other is worked on.  Places past the last
   // token repeat it: their numbers in `coef` make them leave the state alone.
   constexpr int NK = CT * DP * 2 / 4 / 256, NV = (CT * COLS + 255) / 256;
-  float4 rk[NK];
-  float rv[NV];
+  f32x4 rk[NK];
+  float rv[NV], rc[CT / NB], rn[CT / NB];  // rc, rn: the numbers of this stage's blocks and of the next
   auto fetch = [&](int t0) {
 #pragma unroll
     for (int x = 0; x < NK; ++x) {
       const int at = (x * 256 + tid) * 4, t = min(t0 + at / (2 * DP), n - 1);
-      rk[x] = *(const float4 *)(w.qk + ((size_t)(t * a.batch + b) * s.kv_heads + kvh) * 2 * DP + at % (2 * DP));
+      rk[x] = *(const f32x4 *)(w.qk + ((size_t)(t * a.batch + b) * s.kv_heads + kvh) * 2 * DP + at % (2 * DP));
     }
 #pragma unroll
     for (int x = 0; x < NV; ++x) {
       const int at = min(x * 256 + tid, CT * COLS - 1), t = min(t0 + at / COLS, n - 1), cc = min(c0 + at % COLS, V - 1);
       rv[x] = w.raw[(size_t)(t * a.batch + b) * C + 2 * nq + h * V + cc];
     }
+#pragma unroll
+    for (int x = 0; x < CT / NB; ++x) rn[x] = coef[(size_t)min(t0 + x * NB, w.padded - NB) * NCF + min(tid & 63, NB * NCF - 1)];
   };
   auto put = [&](int stage) {
 #pragma unroll
-    for (int x = 0; x < NK; ++x) *(float4 *)(&kq_s[stage][0][0][0] + (x * 256 + tid) * 4) = rk[x];
+    for (int x = 0; x < CT / NB; ++x) rc[x] = rn[x];
+#pragma unroll
+    for (int x = 0; x < NK; ++x) *(f32x4 *)(&kq_s[stage][0][0][0] + (x * 256 + tid) * 4) = rk[x];
 #pragma unroll
     for (int x = 0; x < NV; ++x) {
       const int at = x * 256 + tid;
       if (at < CT * COLS) v_s[stage][at / COLS][at % COLS] = rv[x];
     }
   };
-  Coefs cf[2];
-  cf[0].load(coef);
+  // keys, queries and values of a block, read from LDS while the block before it is worked on
+  float k[2][NB][8], q[2][NB][8], v[2][NB];
+  auto read = [&](int x, int stage, int tb) {
+#pragma unroll
+    for (int j = 0; j < NB; ++j) {
+#pragma unroll
+      for (int half = 0; half < 2; ++half) {
+        const f32x4 kk = *(const f32x4 *)&kq_s[stage][tb + j][0][half * (DP / 2) + l4], qq = *(const f32x4 *)&kq_s[stage][tb + j][1][half * (DP / 2) + l4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          k[x][j][half * 4 + e] = kk[e];
+          q[x][j][half * 4 + e] = qq[e];
+        }
+      }
+      v[x][j] = v_s[stage][tb + j][cl];
+    }
+  };
   fetch(0);
   put(0);
   __syncthreads();
   for (int t0 = 0, stage = 0; t0 < n; t0 += CT, stage ^= 1) {
-    if (t0 + CT < n) fetch(t0 + CT);
+    fetch(t0 + CT);  // past the end: the last token again
+    read(0, stage, 0);
 #pragma unroll
     for (int tb = 0; tb < CT; tb += NB) {
       if (t0 + tb >= n) break;
-      float k[NB][8], v[NB], sk[NB], sq[NB];
+      const int x = (tb / NB) & 1;
+      float sk[NB], sq[NB];
 #pragma unroll
       for (int j = 0; j < NB; ++j) {
-        const float *kp = &kq_s[stage][tb + j][0][r0], *qp = &kq_s[stage][tb + j][1][r0];
-        const float4 ka = *(const float4 *)kp, kb = *(const float4 *)(kp + 4), qa = *(const float4 *)qp, qb = *(const float4 *)(qp + 4);
-        k[j][0] = ka.x; k[j][1] = ka.y; k[j][2] = ka.z; k[j][3] = ka.w; k[j][4] = kb.x; k[j][5] = kb.y; k[j][6] = kb.z; k[j][7] = kb.w;
-        const float q[8] = {qa.x, qa.y, qa.z, qa.w, qb.x, qb.y, qb.z, qb.w};
-        v[j] = v_s[stage][tb + j][cl];
         sk[j] = sq[j] = 0.0f;
 #pragma unroll
         for (int r = 0; r < 8; ++r) {
-          sk[j] = __builtin_fmaf(S[r], k[j][r], sk[j]);
-          sq[j] = __builtin_fmaf(S[r], q[r], sq[j]);
+          sk[j] = __builtin_fmaf(S[r], k[x][j][r], sk[j]);
+          sq[j] = __builtin_fmaf(S[r], q[x][j][r], sq[j]);
         }
       }
+      if (tb + NB < CT) read(x ^ 1, stage, tb + NB);
 #pragma unroll
       for (int j = 0; j < NB; ++j) {
         sk[j] = column_sum<LPC>(sk[j]);
         sq[j] = column_sum<LPC>(sq[j]);
       }
-      // Scalar loads and LDS reads count on one counter and scalar loads come back in any order, so a wait for LDS waits for
-      // them too: the next block's numbers are asked for here, behind this block's last LDS read.
-      __builtin_amdgcn_sched_barrier(0);
-      cf[(tb / NB + 1) & 1].load(coef + (size_t)min(t0 + tb + NB, w.padded - NB) * NCF);
-      __builtin_amdgcn_sched_barrier(0);
-      const Coefs &now = cf[(tb / NB) & 1];
+      Coefs now;
+      now.from_lanes(rc[tb / NB]);
       float u[NB];
 #pragma unroll
       for (int j = 0; j < NB; ++j) {
-        float e = __builtin_fmaf(-now.v[j][CF_GAMMA], sk[j], v[j]), o = now.v[j][CF_GAMMA] * sq[j];
+        float e = __builtin_fmaf(-now.v[j][CF_GAMMA], sk[j], v[x][j]), o = now.v[j][CF_GAMMA] * sq[j];
 #pragma unroll
         for (int d = 1; d <= j; ++d) {
           e = __builtin_fmaf(-now.v[j][CF_KK + d - 1], u[j - d], e);
@@ -350,7 +366,7 @@ __global__ void __launch_bounds__(256) delta_scan_k(KxDeltaArgs a) {
         }
         u[j] = now.v[j][CF_BETA] * e;
         o = __builtin_fmaf(now.v[j][CF_KQ], u[j], o);
-        if (r0 == 0 && col < V && t0 + tb + j < n) a.o[((size_t)((t0 + tb + j) * a.batch + b) * s.heads + h) * V + col] = o;
+        if (l4 == 0) o_s[stage][tb + j][cl] = o;
       }
 #pragma unroll
       for (int r = 0; r < 8; ++r) S[r] *= now.v[NB - 1][CF_GAMMA];
@@ -358,15 +374,21 @@ __global__ void __launch_bounds__(256) delta_scan_k(KxDeltaArgs a) {
       for (int j = 0; j < NB; ++j) {
         const float y = u[j] * now.v[j][CF_END];
 #pragma unroll
-        for (int r = 0; r < 8; ++r) S[r] = __builtin_fmaf(k[j][r], y, S[r]);
+        for (int r = 0; r < 8; ++r) S[r] = __builtin_fmaf(k[x][j][r], y, S[r]);
       }
     }
-    if (t0 + CT < n) put(stage ^ 1);
+    put(stage ^ 1);
     __syncthreads();
+    // the read-outs go to memory here, behind the wait for the next stage's rows, so that no wait is for a store just made
+#pragma unroll
+    for (int x = 0; x < NV; ++x) {
+      const int at = x * 256 + tid, t = t0 + at / COLS, cc = c0 + at % COLS;
+      if (at < CT * COLS && t < n && cc < V) a.o[((size_t)(t * a.batch + b) * s.heads + h) * V + cc] = o_s[stage][at / COLS][at % COLS];
+    }
   }
 #pragma unroll
   for (int r = 0; r < 8; ++r)
-    if (r0 + r < D && col < V) st[(size_t)(r0 + r) * V + col] = S[r];
+    if (row(r) < D && col < V) st[(size_t)row(r) * V + col] = S[r];
 }
 
 }  // namespace

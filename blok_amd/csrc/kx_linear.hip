@@ -29,7 +29,7 @@ template <class T>
 __device__ __forceinline__ void put_glu(const KxLinArgs &a, int t, int col, float g, float u) {
   g = fminf(g, a.limit);
   u = fminf(fmaxf(u, -a.limit), a.limit);
-  ((T *)a.mid)[(size_t)t * a.mid_ld + col] = Elem<T>::make(g * kx_sigmoidf(a.alpha * g) * (u + a.bias));
+  ((T *)a.mid)[(size_t)t * a.mid_ld + col] = Elem<T>::make(g * kxr::sigmoid_for<T>(a.alpha * g) * (u + a.bias));
 }
 // EPI of the kernels: KX_LIN_F32, KX_LIN_GLU, or KX_LIN_STREAMS + number of streams (streams_any: up to KX_MAX_STREAMS)
 constexpr int STREAMS_ANY = KX_LIN_STREAMS + KX_MAX_STREAMS;

@@ -49,6 +49,13 @@ template <> struct Elem<float> {
   }
 };
 
+// sigmoid for a value that is rounded to T next: without branches and with the approximate reciprocal for bf16
+template <class T>
+__device__ __forceinline__ float sigmoid_for(float x) {
+  if constexpr (sizeof(T) == 4) return kx_sigmoidf(x);
+  else return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.44269504088896341f * x));
+}
+
 // sum over the lanes of a wave, in every lane
 __device__ __forceinline__ float wave_sum(float v) {
   float t = v;
@@ -113,7 +120,7 @@ __device__ __forceinline__ void build_row(const KxRowArgs &a, int tok, T *dst, i
       const float sc = kx_rsqrtf(wave_sum(v) / (float)a.vdim + a.eps);
       for (int d = lane; d < a.vdim; d += 64) {
         const int c = h * a.vdim + d;
-        dst[c] = Elem<T>::make(o[c] * sc * a.w[d] * kx_siluf(gate[c]));
+        dst[c] = Elem<T>::make(o[c] * sc * a.w[d] * gate[c] * sigmoid_for<T>(gate[c]));
       }
     }
     for (int c = a.cols + tid; c < ld; c += n) dst[c] = Elem<T>::make(0.0f);

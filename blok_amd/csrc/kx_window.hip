@@ -22,6 +22,7 @@ typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
 typedef float f32x2 __attribute__((ext_vector_type(2)));
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 typedef unsigned int u32x2 __attribute__((ext_vector_type(2)));
+typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
 
 constexpr float NEG_INF = -__builtin_inff();
 constexpr int RB = 4;            // query heads whose values are summed together in win_partial_k
@@ -321,7 +322,7 @@ __global__ void __launch_bounds__(256) win_flash_k(KxWindowArgs a) {
   const int nb0 = seen_blocks(q0, s.size, s.pool), nb1 = seen_blocks(q1, s.size, s.pool), lo0 = window_lo(q0, s.size), lo1 = window_lo(q1, s.size);
   auto first_key = [&](int t) { return t < tb ? t * FK : j0 + (t - tb) * FK; };
   constexpr int VT = (FK / 8) * NV * 16, VN = (VT + 255) / 256;  // V is taken by 8 keys x 2 columns
-  uint4 kreg[ND];
+  u32x4 kreg[ND];
   uint32_t vreg[VN][8];
   // Rows of a tile: a window tile starts at a multiple of FK and the ring's length is one, so it does not wrap inside; past the
   // last block there is nothing to read.  What is read beyond a row's columns or the keys a query sees meets zeros.
@@ -333,7 +334,7 @@ __global__ void __launch_bounds__(256) win_flash_k(KxWindowArgs a) {
 #pragma unroll
     for (int y = 0; y < ND; ++y) {
       const int x = y * 256 + tid, r = x / (ND * 4), d = (x - r * (ND * 4)) * 8;
-      kreg[y] = *(const uint4 *)(kr + (size_t)min(r, last) * c.dp + min(d, c.dp - 8));
+      kreg[y] = *(const u32x4 *)(kr + (size_t)min(r, last) * c.dp + min(d, c.dp - 8));
     }
 #pragma unroll
     for (int y = 0; y < VN; ++y) {
@@ -346,7 +347,7 @@ __global__ void __launch_bounds__(256) win_flash_k(KxWindowArgs a) {
 #pragma unroll
     for (int y = 0; y < ND; ++y) {
       const int x = y * 256 + tid, r = x / (ND * 4), d = (x - r * (ND * 4)) * 8;
-      *(uint4 *)(ks + r * KSTR + d) = kreg[y];
+      *(u32x4 *)(ks + r * KSTR + d) = kreg[y];
     }
 #pragma unroll
     for (int y = 0; y < VN; ++y) {
@@ -369,7 +370,7 @@ __global__ void __launch_bounds__(256) win_flash_k(KxWindowArgs a) {
     __syncthreads();  // the tile before has been multiplied
     put();
     __syncthreads();
-    if (t + 1 < tiles) fetch(t + 1);
+    fetch(min(t + 1, tiles - 1));
     const bool none = pooled ? k0 >= nb1 : k0 > q1 || k0 + FK - 1 < lo0;
     const bool all = pooled ? k0 + FK <= nb0 : k0 >= lo1 && k0 + FK - 1 <= q0;
     if (none) continue;
@@ -384,19 +385,25 @@ __global__ void __launch_bounds__(256) win_flash_k(KxWindowArgs a) {
         sc[kt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, q[kk], sc[kt], 0, 0, 0);
       }
     }
+    const int from = (pooled ? 0 : lo) - k0 - 4 * hh, to = (pooled ? nb - 1 : p) - k0 - 4 * hh;  // the keys this lane's query sees, from its first one on
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+      for (int v = 0; v < 16; ++v) sc[kt][v] *= scale2;
+    if (!all) {
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+        for (int v = 0; v < 16; ++v) {
+          const int e = kt * 32 + 8 * (v >> 2) + (v & 3);
+          sc[kt][v] = ((e < from) | (e > to)) ? NEG_INF : sc[kt][v];
+        }
+    }
     float tm = NEG_INF;
 #pragma unroll
     for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
-      for (int v = 0; v < 16; ++v) {
-        sc[kt][v] *= scale2;
-        if (!all) {
-          const int e = k0 + kt * 32 + 8 * (v >> 2) + 4 * hh + (v & 3);
-          const bool see = pooled ? e < nb : e >= lo && e <= p;
-          sc[kt][v] = see ? sc[kt][v] : NEG_INF;
-        }
-        tm = fmaxf(tm, sc[kt][v]);
-      }
+      for (int v = 0; v < 16; ++v) tm = fmaxf(tm, sc[kt][v]);
     tm = fmaxf(tm, __shfl_xor(tm, 32));
     if (__any(tm > m)) {
       const float m1 = fmaxf(m, tm), al = m == NEG_INF ? 0.0f : __builtin_amdgcn_exp2f(m - m1);
@@ -440,12 +447,19 @@ __global__ void __launch_bounds__(256) win_flash_k(KxWindowArgs a) {
   uint16_t *out = (uint16_t *)a.out + (size_t)tok * a.out_ld + h * s.vdim;
   const float *gate = a.g_off >= 0 ? a.proj + (size_t)tok * a.proj_ld + a.g_off + h * s.vdim : nullptr;
 #pragma unroll
-  for (int j = 0; j < NV; ++j)
+  for (int j = 0; j < NV; ++j) {
+    float gt[16];
+#pragma unroll
+    for (int v = 0; v < 16; ++v) gt[v] = gate ? gate[min(j * 32 + 8 * (v >> 2) + 4 * hh + (v & 3), s.vdim - 1)] : 0.0f;
+#pragma unroll
+    for (int v = 0; v < 16; ++v) asm volatile("" : "+v"(gt[v]));  // all sixteen are asked for before the first is used
 #pragma unroll
     for (int v = 0; v < 16; ++v) {
       const int d = j * 32 + 8 * (v >> 2) + 4 * hh + (v & 3);
-      if (d < s.vdim) out[d] = kx_bf16_rne(o[j][v] * inv * (gate ? kx_sigmoidf(gate[d]) : 1.0f));
+      const float y = o[j][v] * inv * (gate ? kxr::sigmoid_for<uint16_t>(gt[v]) : 1.0f);
+      if (d < s.vdim) out[d] = kx_bf16_rne(y);
     }
+  }
 }
 
 // keys per workgroup of win_partial_k: few parts, but enough workgroups
