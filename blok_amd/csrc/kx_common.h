@@ -31,6 +31,8 @@ void kx_set_error(const char *fmt, ...) __attribute__((format(printf, 1, 2)));
     }                            \
   } while (0)
 
+#define KX_DO(call) do { if (int rc_ = (call)) return rc_; } while (0)
+
 #define KX_LAUNCH_CHECK() KX_HIP(hipGetLastError())
 
 // No exception may cross the C ABI: the host-side entry points that parse files or grow containers run their

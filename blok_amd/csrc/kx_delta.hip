@@ -3,8 +3,8 @@
 // One token per sequence: delta_step_k.  A workgroup owns 32 columns of one head's state; it convolves and norms the
 // head's q and k itself, reads its columns once, and writes them once.
 //
-// Several positions: delta_conv_k (convolutions and silu), delta_unit_k (unit norms and the numbers below),
-// delta_hist_k (the convolutions' inputs that the next step needs) and delta_scan_k, which keeps the state in registers:
+// Several positions: the convolutions (kx_conv.hip), delta_unit_k (unit norms and the numbers below) and delta_scan_k, which
+// keeps the state in registers:
 // the columns of a head's state do not meet, so a column is spread over dim / 8 lanes with 8 rows each, and a wave goes
 // through the tokens.  It takes them in blocks of four, so that the sums over a column's lanes do not wait for each
 // other: with S the state before the block, D(i, j) the product of the decays of tokens i + 1 .. j and D(j) that of tokens
@@ -18,6 +18,7 @@
 #include <algorithm>
 #include <atomic>
 #include "kx_common.h"
+#include "kx_conv.h"
 #include "kx_rows.h"
 #include "kx_delta.h"
 
@@ -27,37 +28,30 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 constexpr int SC = 32;  // columns per workgroup of delta_step_k
 
-// log(1 + exp(x))
-__device__ __forceinline__ float softplus(float x) { return fmaxf(x, 0.0f) + log1pf(kx_expf(-fabsf(x))); }
 __device__ __forceinline__ float decay_of(const KxDeltaArgs &a, const float *pr, int h) {
-  return kx_expf(-kx_expf(a.a_log[h]) * softplus(pr[a.a_off + h] + a.dt_bias[h]));
+  return kx_expf(-kx_expf(a.a_log[h]) * kxr::softplus(pr[a.a_off + h] + a.dt_bias[h]));
 }
 
-// offset in a projection row of convolution channel ch (q, k, v in turn)
-__device__ __forceinline__ int channel_off(const KxDeltaArgs &a, int ch) {
+__host__ __device__ __forceinline__ KxConvArgs conv_of(const KxDeltaArgs &a) {
   const int nq = a.s.kv_heads * a.s.dim;
-  return ch < nq ? a.q_off + ch : ch < 2 * nq ? a.k_off + ch - nq : a.v_off + ch - 2 * nq;
-}
-// input of channel ch at position i of the step (i < 0: before it) of sequence b
-__device__ __forceinline__ float conv_input(const KxDeltaArgs &a, int b, int i, int ch, int off) {
-  return i >= 0 ? a.proj[(size_t)(i * a.batch + b) * a.proj_ld + off]
-                : a.hist[((size_t)b * (a.s.taps - 1) + a.s.taps - 1 + i) * kx_delta_channels(a.s) + ch];
-}
-__device__ __forceinline__ float conv_silu(const KxDeltaArgs &a, int b, int i, int ch) {
-  const int off = channel_off(a, ch);
-  float v = 0.0f;
-  for (int j = 0; j < a.s.taps; ++j) v = __builtin_fmaf(a.conv[(size_t)ch * a.s.taps + j], conv_input(a, b, i - (a.s.taps - 1) + j, ch, off), v);
-  return kx_siluf(v);
+  KxConvArgs c;
+  c.proj = a.proj; c.proj_ld = a.proj_ld;
+  c.segs = 3;
+  c.end[0] = nq; c.end[1] = 2 * nq; c.end[2] = c.channels = kx_delta_channels(a.s);
+  c.off[0] = a.q_off; c.off[1] = a.k_off; c.off[2] = a.v_off;
+  c.taps = a.s.taps; c.w = a.conv;
+  c.hist = a.hist; c.hist_out = a.hist_out; c.batch = a.batch; c.positions = a.positions;
+  return c;
 }
 
-__global__ void __launch_bounds__(256) delta_step_k(KxDeltaArgs a) {
+__global__ void __launch_bounds__(256) delta_step_k(KxDeltaArgs a, KxConvArgs cv) {
   extern __shared__ float dl_lds[];
   __shared__ float red[4];
   __shared__ float part[2][8][SC];
   const KxDeltaSpec &s = a.s;
   const int D = s.dim, V = s.vdim, tid = threadIdx.x, slices = (V + SC - 1) / SC;
   const int h = blockIdx.x / slices, c0 = (blockIdx.x - h * slices) * SC, b = blockIdx.y;
-  const int kvh = h / (s.heads / s.kv_heads), nq = s.kv_heads * D, C = kx_delta_channels(s);
+  const int kvh = h / (s.heads / s.kv_heads), nq = s.kv_heads * D;
   float *q = dl_lds, *k = q + D, *v = k + D, *S = v + SC;  // S [D][SC]
   const int c = tid & (SC - 1), rg = tid / SC, col = min(c0 + c, V - 1);
   float *st = a.state + ((size_t)b * s.heads + h) * D * V;
@@ -66,27 +60,22 @@ __global__ void __launch_bounds__(256) delta_step_k(KxDeltaArgs a) {
   for (int x = tid; x < 2 * D; x += 256) {
     const bool key = x >= D;
     const int d = key ? x - D : x;
-    const float y = conv_silu(a, b, 0, (key ? nq : 0) + kvh * D + d);
+    const float y = kxc::conv_silu(cv, b, 0, (key ? nq : 0) + kvh * D + d);
     (key ? k : q)[d] = y;
     if (key) kk = __builtin_fmaf(y, y, kk);
     else qq = __builtin_fmaf(y, y, qq);
   }
-  if (tid < SC) v[tid] = c0 + tid < V ? conv_silu(a, b, 0, 2 * nq + h * V + c0 + tid) : 0.0f;
+  if (tid < SC) v[tid] = c0 + tid < V ? kxc::conv_silu(cv, b, 0, 2 * nq + h * V + c0 + tid) : 0.0f;
   qq = kxr::block_sum(qq, red);
   kk = kxr::block_sum(kk, red);
   const float qsc = kx_rsqrtf(qq + s.unit_eps) * kx_rsqrtf((float)D), ksc = kx_rsqrtf(kk + s.unit_eps);
   const float *pr = a.proj + (size_t)b * a.proj_ld;
   const float beta = kx_sigmoidf(pr[a.b_off + h]), g = decay_of(a, pr, h);
   // the convolutions' inputs for the next token: this workgroup's value channels, and q and k once per head of theirs
-  const int keep = s.taps - 1;
-  auto shift = [&](int ch) {
-    const int off = channel_off(a, ch);
-    for (int j = 0; j < keep; ++j) a.hist_out[((size_t)b * keep + j) * C + ch] = conv_input(a, b, j - keep + 1, ch, off);
-  };
-  if (keep) {
-    if (tid < SC && c0 + tid < V) shift(2 * nq + h * V + c0 + tid);
+  if (s.taps > 1) {
+    if (tid < SC && c0 + tid < V) kxc::shift(cv, b, 2 * nq + h * V + c0 + tid);
     if (c0 == 0 && h % (s.heads / s.kv_heads) == 0)
-      for (int x = tid; x < 2 * D; x += 256) shift(x < D ? kvh * D + x : nq + kvh * D + x - D);
+      for (int x = tid; x < 2 * D; x += 256) kxc::shift(cv, b, x < D ? kvh * D + x : nq + kvh * D + x - D);
   }
   float sk = 0.0f;
   for (int r = rg; r < D; r += 8) sk = __builtin_fmaf(S[r * SC + c], k[r], sk);
@@ -128,34 +117,6 @@ __host__ __device__ __forceinline__ Work work_of(const KxDeltaArgs &a) {
   w.qk = w.coef + (size_t)a.batch * a.s.heads * w.padded * NCF;
   w.raw = w.qk + (size_t)a.batch * a.positions * a.s.kv_heads * 2 * kx_delta_row(a.s);
   return w;
-}
-
-constexpr int CONV_TOKENS = 16;  // positions a thread of delta_conv_k goes through
-template <int TAPS>              // 0: any number
-__global__ void __launch_bounds__(256) delta_conv_k(KxDeltaArgs a) {
-  const int C = kx_delta_channels(a.s), ch = blockIdx.x * 256 + threadIdx.x, b = blockIdx.z;
-  const int i0 = blockIdx.y * CONV_TOKENS, i1 = min(i0 + CONV_TOKENS, a.positions);
-  if (ch >= C) return;
-  float *raw = work_of(a).raw;
-  if constexpr (TAPS == 0) {
-    for (int i = i0; i < i1; ++i) raw[(size_t)(i * a.batch + b) * C + ch] = conv_silu(a, b, i, ch);
-  } else {
-    const int off = channel_off(a, ch);
-    float w[TAPS], x[CONV_TOKENS + TAPS - 1];
-#pragma unroll
-    for (int j = 0; j < TAPS; ++j) w[j] = a.conv[(size_t)ch * TAPS + j];
-#pragma unroll
-    for (int j = 0; j < TAPS - 1; ++j) x[j] = conv_input(a, b, i0 - (TAPS - 1) + j, ch, off);
-#pragma unroll
-    for (int j = 0; j < CONV_TOKENS; ++j) x[TAPS - 1 + j] = a.proj[(size_t)(min(i0 + j, a.positions - 1) * a.batch + b) * a.proj_ld + off];
-#pragma unroll
-    for (int j = 0; j < CONV_TOKENS; ++j) {
-      float v = 0.0f;
-#pragma unroll
-      for (int t = 0; t < TAPS; ++t) v = __builtin_fmaf(w[t], x[j + t], v);
-      if (i0 + j < i1) raw[(size_t)((i0 + j) * a.batch + b) * C + ch] = kx_siluf(v);
-    }
-  }
 }
 
 // one wave per (position, key head)
@@ -227,14 +188,6 @@ __global__ void __launch_bounds__(256) delta_unit_k(KxDeltaArgs a) {
         if (x == j - d) down *= g[x];
     }
   }
-}
-
-__global__ void __launch_bounds__(256) delta_hist_k(KxDeltaArgs a) {
-  const int C = kx_delta_channels(a.s), keep = a.s.taps - 1, ch = blockIdx.x * 256 + threadIdx.x, b = blockIdx.y;
-  if (ch >= C) return;
-  const int off = channel_off(a, ch);
-  for (int j = 0; j < keep; ++j)
-    a.hist_out[((size_t)b * keep + j) * C + ch] = conv_input(a, b, a.positions - keep + j, ch, off);
 }
 
 template <int LPC>
@@ -401,23 +354,15 @@ int kx_delta_launch(const KxDeltaArgs &a, hipStream_t st) {
   KX_REQUIRE(a.batch > 0 && a.positions > 0 && (s.taps == 1 || (a.hist && a.hist_out && a.hist != a.hist_out)), "delta rule: %d x %d tokens", a.batch, a.positions);
   if (a.positions == 1) {
     const size_t lds = ((size_t)2 * s.dim + SC + (size_t)s.dim * SC) * 4;
-    hipLaunchKernelGGL(delta_step_k, dim3(s.heads * kx_cdiv(s.vdim, SC), a.batch), dim3(256), lds, st, a);
+    hipLaunchKernelGGL(delta_step_k, dim3(s.heads * kx_cdiv(s.vdim, SC), a.batch), dim3(256), lds, st, a, conv_of(a));
     KX_LAUNCH_CHECK();
     return KX_OK;
   }
   KX_REQUIRE(a.work, "delta rule: no scratch");
-  const dim3 conv_grid(kx_cdiv(kx_delta_channels(s), 256), kx_cdiv(a.positions, CONV_TOKENS), a.batch);
-  if (s.taps == 2) hipLaunchKernelGGL(delta_conv_k<2>, conv_grid, dim3(256), 0, st, a);
-  else if (s.taps == 3) hipLaunchKernelGGL(delta_conv_k<3>, conv_grid, dim3(256), 0, st, a);
-  else if (s.taps == 4) hipLaunchKernelGGL(delta_conv_k<4>, conv_grid, dim3(256), 0, st, a);
-  else hipLaunchKernelGGL(delta_conv_k<0>, conv_grid, dim3(256), 0, st, a);
-  KX_LAUNCH_CHECK();
+  const int rc = kx_conv_launch(conv_of(a), work_of(a).raw, st);
+  if (rc) return rc;
   hipLaunchKernelGGL(delta_unit_k, dim3(kx_cdiv(work_of(a).padded * s.kv_heads, 4), a.batch), dim3(256), 0, st, a);
   KX_LAUNCH_CHECK();
-  if (s.taps > 1) {
-    hipLaunchKernelGGL(delta_hist_k, dim3(kx_cdiv(kx_delta_channels(s), 256), a.batch), dim3(256), 0, st, a);
-    KX_LAUNCH_CHECK();
-  }
 #define KX_SCAN(LPC) hipLaunchKernelGGL(delta_scan_k<LPC>, dim3(kx_cdiv(s.vdim, 256 / LPC), s.heads, a.batch), dim3(256), 0, st, a)
   if (s.dim <= 32) KX_SCAN(4);
   else if (s.dim <= 64) KX_SCAN(8);

@@ -115,8 +115,9 @@ __global__ void __launch_bounds__(PART_THREADS) win_partial_k(KxWindowArgs a, in
   float *qv = win_lds;                 // [R][dp]
   float *sc = qv + R * c.dp;           // [R][ch]
   float *sum = sc + R * ch;            // [groups][RB][vp]
-  const size_t head = (size_t)b * s.kv_heads + g;
-  const T *kc = (const T *)c.k + head * c.cap * c.dp, *vc = (const T *)c.v + head * c.cap * c.vp;
+  const size_t head = c.shared ? b : (size_t)b * s.kv_heads + g;
+  const int kld = c.k_ld ? c.k_ld : c.dp, vld = c.v_ld ? c.v_ld : c.vp;
+  const T *kc = (const T *)c.k + head * c.cap * kld, *vc = (const T *)c.v + head * c.cap * vld;
   const T *pkc = (const T *)c.pk + head * c.blocks * c.dp, *pvc = (const T *)c.pv + head * c.blocks * c.vp;
   if (FUSED) {
     const float *pr = a.proj + (size_t)tok * a.proj_ld;
@@ -148,8 +149,11 @@ __global__ void __launch_bounds__(PART_THREADS) win_partial_k(KxWindowArgs a, in
       if (s.pool > 0 && (p + 1) % s.pool == 0 && p / s.pool < c.blocks) pool_block<T>(a, head, p / s.pool, tid, PART_THREADS);
     }
   } else {
-    const T *q = (const T *)a.q + ((size_t)tok * s.heads + g * R) * c.dp;
-    for (int x = tid; x < R * c.dp; x += PART_THREADS) qv[x] = E::load(q + x);
+    const size_t q0 = ((size_t)tok * s.heads + g * R) * c.dp;
+    if (a.q_f32)
+      for (int x = tid; x < R * c.dp; x += PART_THREADS) qv[x] = a.q_f32[q0 + x];
+    else
+      for (int x = tid; x < R * c.dp; x += PART_THREADS) qv[x] = E::load((const T *)a.q + q0 + x);
   }
   __syncthreads();
   const int base = p / c.cap * c.cap;  // position j of the window: slot j - base, one ring length more below it
@@ -161,7 +165,7 @@ __global__ void __launch_bounds__(PART_THREADS) win_partial_k(KxWindowArgs a, in
   const int l8 = lane & 7;
   for (int k0 = wave * 8; k0 < n; k0 += 32) {
     const int e = e0 + min(k0 + (lane >> 3), n - 1);
-    const T *key = e < nb ? pkc + (size_t)e * c.dp : kc + (size_t)slot_of(e) * c.dp;
+    const T *key = e < nb ? pkc + (size_t)e * c.dp : kc + (size_t)slot_of(e) * kld;
     for (int r0 = 0; r0 < R; r0 += RB) {
       float d[RB] = {};
       for (int x = l8 * 8; x < c.dp; x += 64) {
@@ -211,7 +215,7 @@ __global__ void __launch_bounds__(PART_THREADS) win_partial_k(KxWindowArgs a, in
       for (int k = grp; k < n; k += groups) {
         const int e = e0 + k;
         float vf[8];
-        E::unpack(vf, E::cached((e < nb ? pvc + (size_t)e * c.vp : vc + (size_t)slot_of(e) * c.vp) + col));
+        E::unpack(vf, E::cached((e < nb ? pvc + (size_t)e * c.vp : vc + (size_t)slot_of(e) * vld) + col));
 #pragma unroll
         for (int r = 0; r < RB; ++r) {
           const float w = sc[min(r0 + r, R - 1) * ch + k];
@@ -245,7 +249,8 @@ __global__ void __launch_bounds__(MERGE_THREADS) win_merge_k(KxWindowArgs a, int
   const int h = blockIdx.x, tok = tok0 + blockIdx.y, tid = threadIdx.x;
   const size_t row = (size_t)blockIdx.y * parts;
   if (tid < 64) {
-    float m = s.sink ? 0.0f : NEG_INF, z = 0.0f;
+    const float sink = a.sinks ? a.sinks[h] : 0.0f;
+    float m = s.sink ? sink : NEG_INF, z = 0.0f;
     for (int k = tid; k < parts; k += 64) m = fmaxf(m, pm[(row + k) * s.heads + h]);
     m = kxw::wave_max_f32(m);
     for (int k = tid; k < parts; k += 64) {
@@ -253,7 +258,7 @@ __global__ void __launch_bounds__(MERGE_THREADS) win_merge_k(KxWindowArgs a, int
       weight[k] = w;
       z = __builtin_fmaf(pz[(row + k) * s.heads + h], w, z);
     }
-    const float inv = 1.0f / (kxr::wave_sum(z) + (s.sink ? kx_expf(-m) : 0.0f));
+    const float inv = 1.0f / (kxr::wave_sum(z) + (s.sink ? kx_expf(sink - m) : 0.0f));
     for (int k = tid; k < parts; k += 64) weight[k] *= inv;
   }
   __syncthreads();
@@ -310,7 +315,7 @@ __global__ void __launch_bounds__(256) win_flash_k(KxWindowArgs a) {
   for (int j = 0; j < NV; ++j)
 #pragma unroll
     for (int v = 0; v < 16; ++v) o[j][v] = 0.0f;
-  float m = s.sink ? 0.0f : NEG_INF, z = s.sink && hh == 0 ? 1.0f : 0.0f;  // z: this lane's half of the keys
+  float m = s.sink ? (a.sinks ? a.sinks[h] * 1.44269504088896341f : 0.0f) : NEG_INF, z = s.sink && hh == 0 ? 1.0f : 0.0f;  // z: this lane's half of the keys
   const float scale2 = s.scale * 1.44269504088896341f;
 
   // tiles: the blocks the last query sees, then the positions from the first query's window on
@@ -492,34 +497,22 @@ int flash_nv(const KxWindowArgs &a, int nv, hipStream_t st) {
   return KX_OK;
 }
 
-template <class T>
-int attention(const KxWindowArgs &a, hipStream_t st) {
+int check(const KxWindowArgs &a) {
   const KxWindowSpec &s = a.s;
-  const int tokens = a.batch * a.positions, R = s.heads / s.kv_heads;
   KX_REQUIRE(s.heads > 0 && s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.dim > 0 && s.vdim > 0 && s.size > 0 && s.pool >= 0,
              "window attention: heads=%d kv_heads=%d dim=%d vdim=%d size=%d pool=%d", s.heads, s.kv_heads, s.dim, s.vdim, s.size, s.pool);
   KX_REQUIRE(a.c.vp <= 2048, "window attention: values of %d columns", s.vdim);
-  KX_REQUIRE(tokens > 0 && a.pos >= 0, "window attention: %d tokens at position %d", tokens, a.pos);
-  const bool fused = a.positions == 1;
-  if (!fused) {
-    hipLaunchKernelGGL((win_prep_k<T>), dim3(tokens), dim3(256), 0, st, a);
-    KX_LAUNCH_CHECK();
-    if (s.pool > 0) {  // blocks whose last position is in this step
-      const int b0 = a.pos / s.pool, b1 = std::min((a.pos + a.positions) / s.pool, a.c.blocks);
-      if (b1 > b0) {
-        hipLaunchKernelGGL((win_pool_k<T>), dim3(b1 - b0, s.kv_heads, a.batch), dim3(256), 0, st, a, b0);
-        KX_LAUNCH_CHECK();
-      }
-    }
-    if (sizeof(T) == 2 && a.c.dp <= 256 && a.c.vp <= 256) {
-      const int nd = a.c.dp / 32, nv = a.c.vp / 32;
-      return nd == 1 ? flash_nv<1>(a, nv, st) : nd == 2 ? flash_nv<2>(a, nv, st) : nd <= 4 ? flash_nv<4>(a, nv, st) : flash_nv<8>(a, nv, st);
-    }
-  }
-  const int total = most_keys(s, a.pos + a.positions), ch = part_keys(s, total, tokens), parts = kx_cdiv(total, ch);
+  KX_REQUIRE(a.batch > 0 && a.positions > 0 && a.pos >= 0, "window attention: %d x %d tokens at position %d", a.batch, a.positions, a.pos);
+  return KX_OK;
+}
+
+template <class T>
+int parts_launch(const KxWindowArgs &a, bool fused, int tok0, int tokens, KxWindowParts &out, hipStream_t st) {
+  const KxWindowSpec &s = a.s;
+  const int R = s.heads / s.kv_heads, total = most_keys(s, a.pos + a.positions), ch = part_keys(s, total, tokens), parts = kx_cdiv(total, ch);
   const size_t per_token = (size_t)parts * floats_per_part(s);
   KX_REQUIRE(per_token <= a.part_floats, "window attention: %zu floats of partials, room for %zu", per_token, a.part_floats);
-  const int at_once = (int)std::min<size_t>({(size_t)tokens, a.part_floats / per_token, (size_t)65535});
+  const int n = (int)std::min<size_t>({(size_t)tokens, a.part_floats / per_token, (size_t)65535});
   const size_t lds = ((size_t)R * a.c.dp + (size_t)R * ch + (size_t)(PART_THREADS / (a.c.vp / 8)) * RB * a.c.vp) * 4;
   KX_REQUIRE(lds <= 160 * 1024 - 256, "window attention: %d query heads of %d per key head do not fit a workgroup", R, s.dim);
   static std::atomic<bool> attr{false};
@@ -528,17 +521,56 @@ int attention(const KxWindowArgs &a, hipStream_t st) {
     KX_HIP(hipFuncSetAttribute((const void *)win_partial_k<T, false>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 256));
     attr = true;
   }
-  for (int t0 = 0; t0 < tokens; t0 += at_once) {
-    const int n = std::min(at_once, tokens - t0);
-    float *po = a.part, *pm = po + (size_t)n * parts * s.heads * a.c.vp, *pz = pm + (size_t)n * parts * s.heads;
-    const dim3 grid(parts, s.kv_heads, n);
-    if (fused) hipLaunchKernelGGL((win_partial_k<T, true>), grid, dim3(PART_THREADS), lds, st, a, t0, ch, po, pm, pz);
-    else hipLaunchKernelGGL((win_partial_k<T, false>), grid, dim3(PART_THREADS), lds, st, a, t0, ch, po, pm, pz);
-    KX_LAUNCH_CHECK();
-    hipLaunchKernelGGL((win_merge_k<T>), dim3(s.heads, n), dim3(MERGE_THREADS), (size_t)parts * 4, st, a, t0, parts, po, pm, pz);
+  float *po = a.part, *pm = po + (size_t)n * parts * s.heads * a.c.vp, *pz = pm + (size_t)n * parts * s.heads;
+  const dim3 grid(parts, s.kv_heads, n);
+  if (fused) hipLaunchKernelGGL((win_partial_k<T, true>), grid, dim3(PART_THREADS), lds, st, a, tok0, ch, po, pm, pz);
+  else hipLaunchKernelGGL((win_partial_k<T, false>), grid, dim3(PART_THREADS), lds, st, a, tok0, ch, po, pm, pz);
+  KX_LAUNCH_CHECK();
+  out.n = n; out.parts = parts; out.o = po; out.m = pm; out.z = pz;
+  return KX_OK;
+}
+
+// parts and merge
+template <class T>
+int attend_parts(const KxWindowArgs &a, bool fused, hipStream_t st) {
+  const int tokens = a.batch * a.positions;
+  KxWindowParts p;
+  for (int t0 = 0; t0 < tokens; t0 += p.n) {
+    int rc = parts_launch<T>(a, fused, t0, tokens - t0, p, st);
+    if (rc) return rc;
+    hipLaunchKernelGGL((win_merge_k<T>), dim3(a.s.heads, p.n), dim3(MERGE_THREADS), (size_t)p.parts * 4, st, a, t0, p.parts, p.o, p.m, p.z);
     KX_LAUNCH_CHECK();
   }
   return KX_OK;
+}
+
+// queries and cache rows in place
+template <class T>
+int attend(const KxWindowArgs &a, hipStream_t st) {
+  if (sizeof(T) == 2 && a.c.dp <= 256 && a.c.vp <= 256) {
+    const int nd = a.c.dp / 32, nv = a.c.vp / 32;
+    return nd == 1 ? flash_nv<1>(a, nv, st) : nd == 2 ? flash_nv<2>(a, nv, st) : nd <= 4 ? flash_nv<4>(a, nv, st)
+         : nd <= 6 ? flash_nv<6>(a, nv, st) : flash_nv<8>(a, nv, st);
+  }
+  return attend_parts<T>(a, false, st);
+}
+
+template <class T>
+int attention(const KxWindowArgs &a, hipStream_t st) {
+  const KxWindowSpec &s = a.s;
+  int rc = check(a);
+  if (rc) return rc;
+  if (a.positions == 1) return attend_parts<T>(a, true, st);
+  hipLaunchKernelGGL((win_prep_k<T>), dim3(a.batch * a.positions), dim3(256), 0, st, a);
+  KX_LAUNCH_CHECK();
+  if (s.pool > 0) {  // blocks whose last position is in this step
+    const int b0 = a.pos / s.pool, b1 = std::min((a.pos + a.positions) / s.pool, a.c.blocks);
+    if (b1 > b0) {
+      hipLaunchKernelGGL((win_pool_k<T>), dim3(b1 - b0, s.kv_heads, a.batch), dim3(256), 0, st, a, b0);
+      KX_LAUNCH_CHECK();
+    }
+  }
+  return attend<T>(a, st);
 }
 
 }  // namespace
@@ -562,3 +594,12 @@ size_t kx_window_part_floats(const KxWindowSpec &s, int max_context, int tokens)
 }
 
 int kx_window_launch(bool f32, const KxWindowArgs &a, hipStream_t st) { return f32 ? attention<float>(a, st) : attention<uint16_t>(a, st); }
+
+int kx_window_attend(bool f32, const KxWindowArgs &a, hipStream_t st) {
+  const int rc = check(a);
+  return rc ? rc : f32 ? attend<float>(a, st) : attend<uint16_t>(a, st);
+}
+int kx_window_parts_launch(bool f32, const KxWindowArgs &a, int tok0, int tokens, KxWindowParts *out, hipStream_t st) {
+  const int rc = check(a);
+  return rc ? rc : f32 ? parts_launch<float>(a, false, tok0, tokens, *out, st) : parts_launch<uint16_t>(a, false, tok0, tokens, *out, st);
+}
