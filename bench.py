@@ -11,7 +11,7 @@ already resident in HBM.  Workloads:
   moe_layer : config 2 alone, one routed-MoE decode layer at Kimi-K2 shape for `--tokens`
               tokens.  Weights of several independent layers are cycled so that neither L2
               nor the 256 MB Infinity Cache can serve them.
-  hybrid    : the Kagalorn design at the layer sizes of real models (random weights), prefill and decode, each beside a
+  hybrid    : the Rapitar and Kagalorn designs at the layer sizes of real models (random weights), prefill and decode, beside a
               Kimi-K2 stack of dense layers of the same hidden size, heads and feed-forward.
 Prints ONE JSON line.
 """
@@ -708,6 +708,46 @@ def hybrid_config(size):
             "layers": [attn, delta] * (HYBRID_LAYERS // 2)}
 
 
+# the Rapitar design at the same widths: state-space layers of twice the width in heads of 64, time mixing in heads of 64, latent
+# attention in heads of 128 + 64; half the layers have a plain feed-forward, half RAPITAR_TOP of RAPITAR_EXPERTS experts
+RAPITAR_EXPERTS, RAPITAR_TOP, RAPITAR_STATE, RAPITAR_RANKS = 64, 8, 128, (1536, 512)     # RANKS: of queries, of keys and values
+
+
+def rapitar_config(size):
+    width, heads, kv, ff = HYBRID_SIZES[size]
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "expert": {"ff": ff // RAPITAR_TOP}, "router": {"experts": RAPITAR_EXPERTS, "top": RAPITAR_TOP}}
+    ssd = {"heads": 2 * width // 64, "vdim": 64, "state": RAPITAR_STATE, "groups": kv, "norm_groups": kv, "conv": 4}
+    wkv = {"heads": width // 64, "dim": 64}
+    latent = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": RAPITAR_RANKS[0], "kv_rank": RAPITAR_RANKS[1], "scale": 192 ** -0.5,
+              "rot": {"dims": 64, "base": 10000.0}}
+    four = [("mamba2", ssd, dense), ("wkv", wkv, moe), ("latent_attention", latent, dense), ("mamba2", ssd, moe)]
+    return {"architecture": "Rapitar", "vocab": HYBRID_VOCAB, "width": width, "norm": {"eps": 1e-5},
+            "layers": [{"type": t, "mixer": m, "mlp": f} for t, m, f in four] * (HYBRID_LAYERS // 4)}
+
+
+def rapitar_counts(size, P):
+    """(weights a token meets, cache and state bytes of a decoded token)"""
+    width, heads, kv, ff = HYBRID_SIZES[size]
+    params = state = 0
+    for layer in rapitar_config(size)["layers"]:
+        m = layer["mixer"]
+        if layer["type"] == "mamba2":
+            inner, bc = m["heads"] * m["vdim"], 2 * m["groups"] * m["state"]
+            params += width * (2 * inner + bc + m["heads"]) + width * inner
+            state += m["heads"] * m["vdim"] * m["state"] * 4 * 2
+        elif layer["type"] == "wkv":
+            hd = m["heads"] * m["dim"]
+            params += 5 * width * hd + 64 * (width + hd)
+            state += hd * m["dim"] * 4 * 2
+        else:
+            hd, r = m["heads"], m["kv_rank"]
+            params += width * (m["q_rank"] + r + m["rot_dim"] + 2 * hd * m["vdim"]) + m["q_rank"] * hd * (m["dim"] + m["rot_dim"]) + r * hd * (m["dim"] + m["vdim"])
+            state += P * (r + m["rot_dim"]) * 2
+        params += 2 * width * ff if layer["mlp"]["kind"] == "dense" else 3 * width * ff + RAPITAR_EXPERTS * width
+    return params, state
+
+
 def timed_model(lib, model, prompt, P, chunk, K, W, vocab):
     """ms per prefill of a P-token prompt and per decode step after it (batch 1, greedy, ids stay on the device); the best of
     three prefills, so that the first one's code loading does not count."""
@@ -742,20 +782,24 @@ def hybrid_leg(lib, size, design, P, K, W, seed, chunk):
     from blok_amd.lib import KxOpenOptions, check, default_config
     width, heads, kv, ff = HYBRID_SIZES[size]
     model = C.c_void_p()
-    if design == "kagalorn":
+    if design in ("kagalorn", "rapitar"):
         o = KxOpenOptions()
         check(lib.kx_open_options_default(C.byref(o)))
         o.max_context, o.random_init, o.seed, o.step_tokens = P + K + W + 1, 1, seed, chunk
         with tempfile.TemporaryDirectory() as d:
             with open(os.path.join(d, "config.json"), "w") as f:
-                json.dump(hybrid_config(size), f)
+                json.dump({"kagalorn": hybrid_config, "rapitar": rapitar_config}[design](size), f)
             check(lib.kx_model_open(d.encode(), C.byref(o), C.byref(model)))
+    if design == "kagalorn":
         hd = heads * HYBRID_DIM
         attn = width * (hd + 2 * kv * HYBRID_DIM + hd + hd)              # q, k, v, gate, output
         delta = width * (2 * (heads // 2) * HYBRID_DIM + 3 * hd + 2 * heads)
         layer = [attn, delta] * (HYBRID_LAYERS // 2)
         keys = HYBRID_WINDOW + max(0, P - HYBRID_WINDOW) // HYBRID_POOL
         state = HYBRID_LAYERS // 2 * (keys * kv * 2 * HYBRID_DIM * 2 + heads * HYBRID_DIM * HYBRID_DIM * 4 * 2)   # cache rows read, state read and written
+        params = sum(layer) + HYBRID_LAYERS * 3 * ff * width
+    elif design == "rapitar":
+        params, state = rapitar_counts(size, P)
     else:
         c = default_config()
         c.n_layers = c.first_dense = HYBRID_LAYERS
@@ -765,7 +809,7 @@ def hybrid_leg(lib, size, design, P, K, W, seed, chunk):
         layer = [width * (c.q_rank + kva) + heads * (c.qk_nope + c.qk_rope) * c.q_rank + heads * (c.qk_nope + c.v_head) * c.kv_rank
                  + width * heads * c.v_head] * HYBRID_LAYERS
         state = HYBRID_LAYERS * P * kva * 2
-    params = sum(layer) + HYBRID_LAYERS * 3 * ff * width
+        params = sum(layer) + HYBRID_LAYERS * 3 * ff * width
     prompt = device_tokens(lib, P, seed, HYBRID_VOCAB)
     pre, dec = timed_model(lib, model, prompt, P, chunk, K, W, HYBRID_VOCAB)
     check(lib.kx_model_destroy(model))
@@ -802,7 +846,7 @@ def main():
     ap.add_argument("--warmup", type=int, default=8)
     ap.add_argument("--workload", default="stack", choices=["stack", "moe_layer", "prefill", "mla", "copy", "load", "hybrid"])
     ap.add_argument("--hybrid-size", default=None, help="hybrid: sizes to run, with commas (default: all)")
-    ap.add_argument("--hybrid-designs", default="kagalorn,kimi_dense", help="hybrid: designs to run")
+    ap.add_argument("--hybrid-designs", default="rapitar,kagalorn,kimi_dense", help="hybrid: designs to run")
     ap.add_argument("--load-dir", default=None, help="where the load workload writes its sparse shards (default: the temp dir)")
     ap.add_argument("--context", type=int, default=32768)
     ap.add_argument("--copy-mib", type=int, default=1024)

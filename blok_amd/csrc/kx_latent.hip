@@ -4,21 +4,29 @@
 // a sink and an output gate; kx_mla.hip is the same for Kimi-K2's.
 //
 // Few positions: W_uk is applied to the query (absorb_k, which also writes the cache rows), so that all heads attend to the
-// cached rows themselves (kx_window.hip: one set of rows for groups of heads, values the first columns of the keys), and
-// latent_out_k merges the parts, applies W_uv and the gate.
+// cached rows themselves: latent_part_k takes tiles of them into LDS once for a group of heads, keys and, in their first
+// columns, values; latent_out_k merges the parts, applies W_uv and the gate.
 // Longer steps: prep_k writes queries and cache rows, two products make the keys and values of every position up to the
 // step's last one, and kx_window.hip attends on the matrix cores.
 #include <math.h>
 #include <algorithm>
+#include <atomic>
 #include <vector>
 #include "kx_common.h"
 #include "kx_latent.h"
+#include "kx_lds_copy.h"
 #include "kx_rows.h"
 
 namespace {
 
 using kxr::Elem;
-constexpr int ABS_COLS = 128, OUT_ROWS = 32, HEAD_GROUP = 8;
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+constexpr int ABS_COLS = 128, OUT_ROWS = 32;
+constexpr int GROUP = 8, KEYS = 64;             // heads of a workgroup of latent_part_k, keys of a tile
+constexpr int MAX_PARTS = 1024;
+constexpr size_t PART_LDS = 78 * 1024;  // two workgroups per CU, where a tile of 16 keys allows
+constexpr size_t MOST_LDS = 158 * 1024;
 constexpr size_t EXPAND_BYTES = (size_t)8 << 30;  // most memory for the keys (and as much for the values) of a step's context
 
 int window_row(const KxLatentSpec &s) { return kx_pad(s.kv_rank + s.rot_dim, 32); }
@@ -93,43 +101,229 @@ __global__ void __launch_bounds__(256) absorb_k(KxLatentArgs a, int row) {
   }
 }
 
+struct Parts {
+  int n, parts, per, keys;  // tokens of the launch; parts per token, tiles per part, keys per tile
+  float *o, *m, *z;         // [n][parts][heads][vp] sums, [n][parts][heads] maxima, denominators
+};
+
+// Part blockIdx.x of the keys of token tok0 + blockIdx.z for the heads of group blockIdx.y: p.per tiles of p.keys keys.  A
+// tile's rows go from memory to LDS whole, the 16-byte pieces of row r at place piece ^ (r % 8), so that lanes on
+// neighbouring rows read different banks.  A lane scores a key (f32) or four keys of a head on the matrix cores (bf16);
+// then a thread owns 2 NC columns of all heads' sums.
+template <class T, int NC>
+__global__ void __launch_bounds__(256) latent_part_k(KxLatentArgs a, Parts p, int tok0, int row, int vp) {
+  constexpr int PE = 16 / sizeof(T);  // elements per piece
+  constexpr bool MC = sizeof(T) == 2;
+  extern __shared__ __attribute__((aligned(16))) uint8_t lp_lds[];
+  const KxLatentSpec &s = a.s;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int tok = tok0 + blockIdx.z, i = tok / a.batch, b = tok - i * a.batch, total = a.pos + i + 1;
+  const int ld = kx_pad(s.kv_rank + s.rot_dim, KX_LD), pieces = ld / PE, qs_ld = row + 8, h0 = blockIdx.y * GROUP, heads = min(GROUP, s.heads - h0);
+  T *tile = (T *)lp_lds;                                       // [keys][ld]
+  T *qs = tile + (size_t)p.keys * ld;                          // [GROUP][row + 8]
+  float *sc = (float *)(qs + (size_t)GROUP * qs_ld), *st_m = sc + GROUP * KEYS, *st_a = st_m + GROUP;
+  const size_t out0 = ((size_t)blockIdx.z * p.parts + blockIdx.x) * s.heads + h0;
+  const int first = blockIdx.x * p.per * p.keys;
+  if (first >= total) {  // fewer keys than the launch's largest token has
+    if (tid < heads) {
+      p.m[out0 + tid] = -__builtin_inff();
+      p.z[out0 + tid] = 0.0f;
+    }
+    return;
+  }
+  const uint32_t lds0 = (uint32_t)(uintptr_t)(__attribute__((address_space(3))) uint8_t *)lp_lds;
+  const T *rows = (const T *)a.rows + (size_t)b * a.cap * ld;
+  const float *q = a.x.q + ((size_t)tok * s.heads + h0) * row;
+  float acc[NC * 2][GROUP] = {};
+  float m[2] = {-__builtin_inff(), -__builtin_inff()}, z[2] = {0.0f, 0.0f};  // of heads wave, wave + 4
+  for (int t = 0; t < p.per; ++t) {
+    const int k0 = first + t * p.keys, n = min(p.keys, total - k0);
+    if (n <= 0) break;
+    if (t) __syncthreads();  // the tile before is done with
+    for (int x = wave * 64; x < p.keys * pieces; x += 256) {
+      const int at = x + lane, r = at / pieces, c = at - r * pieces;
+      kx_copy16_to_lds(rows + (size_t)(k0 + min(r, n - 1)) * ld + (c ^ (r & 7)) * PE, __builtin_amdgcn_readfirstlane(lds0 + x * 16));
+    }
+    if (t == 0)
+#pragma unroll 5
+      for (int x = tid; x < GROUP * row / 4; x += 256) {  // heads lie one after the other
+        const int r = 4 * x / row, d = 4 * x - r * row;
+        const f32x4 y = *(const f32x4 *)(q + 4 * min(x, heads * row / 4 - 1));
+#pragma unroll
+        for (int e = 0; e < 4; ++e) qs[r * qs_ld + d + e] = Elem<T>::make(r < heads ? y[e] : 0.0f);
+      }
+    kx_wait_copies<0>();
+    __syncthreads();
+    if constexpr (MC) {
+      const int lk = lane & 15, g = lane >> 4;
+      for (int kb = wave * 16; kb < p.keys; kb += 64) {
+        f32x4 d[2] = {{0.0f, 0.0f, 0.0f, 0.0f}, {0.0f, 0.0f, 0.0f, 0.0f}};
+        const T *kr = tile + (size_t)(kb + lk) * ld;
+        int x = 0;
+        for (; x + 64 <= row; x += 64)
+#pragma unroll
+          for (int y = 0; y < 2; ++y) {
+            const bf16x8 kf = *(const bf16x8 *)(kr + ((x / 8 + 4 * y + g) ^ (lk & 7)) * 8), qf = *(const bf16x8 *)(qs + (lk & 7) * qs_ld + x + 32 * y + 8 * g);
+            d[y] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf, d[y], 0, 0, 0);
+          }
+        if (x < row) {
+          const bf16x8 kf = *(const bf16x8 *)(kr + ((x / 8 + g) ^ (lk & 7)) * 8), qf = *(const bf16x8 *)(qs + (lk & 7) * qs_ld + x + 8 * g);
+          d[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf, d[0], 0, 0, 0);
+        }
+        if (lk < GROUP) *(f32x4 *)(sc + lk * KEYS + kb + 4 * g) = (d[0] + d[1]) * s.scale;
+      }
+    } else {
+      float d[2] = {};
+      const T *kr = tile + (size_t)min(lane, p.keys - 1) * ld;
+      for (int x = 0; x < row; x += 4) {
+        const f32x4 kf = *(const f32x4 *)(kr + ((x / 4) ^ (lane & 7)) * 4);
+#pragma unroll
+        for (int y = 0; y < 2; ++y) {
+          const f32x4 qf = *(const f32x4 *)(qs + (wave + 4 * y) * qs_ld + x);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) d[y] = __builtin_fmaf(kf[e], qf[e], d[y]);
+        }
+      }
+      if (lane < p.keys)
+#pragma unroll
+        for (int y = 0; y < 2; ++y) sc[(wave + 4 * y) * KEYS + lane] = d[y] * s.scale;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int y = 0; y < 2; ++y) {
+      const int h = wave + 4 * y;
+      const float v = lane < n ? sc[h * KEYS + lane] : -__builtin_inff(), m1 = fmaxf(m[y], kxw::wave_max_f32(v)), al = kx_expf(m[y] - m1);
+      const float e = lane < n ? kx_expf(v - m1) : 0.0f;
+      sc[h * KEYS + lane] = e;
+      z[y] = z[y] * al + kxr::wave_sum(e);
+      m[y] = m1;
+      if (lane == 0) st_a[h] = al;
+    }
+    __syncthreads();
+    float al[GROUP];
+#pragma unroll
+    for (int h = 0; h < GROUP; ++h) al[h] = t ? st_a[h] : 1.0f;
+#pragma unroll
+    for (int c = 0; c < NC * 2; ++c)
+#pragma unroll
+      for (int h = 0; h < GROUP; ++h) acc[c][h] *= al[h];
+    for (int k = 0; k < n; k += 4) {
+      f32x4 wt[GROUP];
+#pragma unroll
+      for (int h = 0; h < GROUP; ++h) wt[h] = *(const f32x4 *)(sc + h * KEYS + k);
+#pragma unroll
+      for (int kk = 0; kk < 4; ++kk) {
+        const T *kr = tile + (size_t)min(k + kk, p.keys - 1) * ld;
+#pragma unroll
+        for (int c = 0; c < NC; ++c) {
+          const int col = c * 512 + tid * 2;
+          float v0 = 0.0f, v1 = 0.0f;
+          if (col < vp) {
+            const T *x = kr + ((col / PE) ^ ((k + kk) & 7)) * PE + col % PE;
+            if constexpr (MC) {
+              const uint32_t two = *(const uint32_t *)x;
+              v0 = kx_bits_f32(two << 16);
+              v1 = kx_bits_f32(two & 0xffff0000u);
+            } else {
+              v0 = x[0];
+              v1 = x[1];
+            }
+          }
+#pragma unroll
+          for (int h = 0; h < GROUP; ++h) {
+            acc[2 * c][h] = __builtin_fmaf(wt[h][kk], v0, acc[2 * c][h]);
+            acc[2 * c + 1][h] = __builtin_fmaf(wt[h][kk], v1, acc[2 * c + 1][h]);
+          }
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int col = c * 512 + tid * 2;
+    if (col < vp)
+#pragma unroll
+      for (int h = 0; h < GROUP; ++h)
+        if (h < heads) *(float2 *)(p.o + (out0 + h) * vp + col) = make_float2(acc[2 * c][h], acc[2 * c + 1][h]);
+  }
+#pragma unroll
+  for (int y = 0; y < 2; ++y)
+    if (lane == 0 && wave + 4 * y < heads) {
+      p.m[out0 + wave + 4 * y] = m[y];
+      p.z[out0 + wave + 4 * y] = z[y];
+    }
+}
+
 // the parts of one head of one token merged with the sink, OUT_ROWS rows of its W_uv, the gate
+constexpr int OUT_THREADS = 512, OUT_AHEAD = 20;  // OUT_AHEAD: a thread's parts that are asked for before the weights are known
 template <class T>
-__global__ void __launch_bounds__(256) latent_out_k(KxLatentArgs a, KxWindowParts w, int tok0, int vp) {
+__global__ void __launch_bounds__(OUT_THREADS) latent_out_k(KxLatentArgs a, Parts w, int tok0, int vp) {
   using E = Elem<T>;
-  extern __shared__ float lo_lds[];
+  extern __shared__ __attribute__((aligned(16))) float lo_lds[];
   const KxLatentSpec &s = a.s;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, slices = (s.vdim + OUT_ROWS - 1) / OUT_ROWS;
   const int h = blockIdx.x / slices, v0 = (blockIdx.x - h * slices) * OUT_ROWS, tok = tok0 + blockIdx.y, ld = a.uv.ld;
-  float *lat = lo_lds, *weight = lat + ld;  // [ld], [parts]
+  float *lat = lo_lds, *sum = lat + ld, *weight = sum + 4 * ld, *den = weight + w.parts;  // [ld], [4][ld], [parts], [parts]
   const size_t row = (size_t)blockIdx.y * w.parts;
+  // four columns per thread; where fewer threads hold them all, the others take parts of their own
+  const int quads = vp / 4, shares = quads <= OUT_THREADS / 4 ? 4 : quads <= OUT_THREADS / 2 ? 2 : 1, per = OUT_THREADS / shares, share = tid / per, tq = tid - share * per;
+  const float *po = w.o + (row * s.heads + h) * vp;
+  auto part = [&](int k, int x) { return *(const f32x4 *)(po + (size_t)min(k, w.parts - 1) * s.heads * vp + 4 * min(x, quads - 1)); };
+  f32x4 y[OUT_AHEAD];
+#pragma unroll
+  for (int j = 0; j < OUT_AHEAD; ++j) y[j] = part(share + j * shares, tq);
+  constexpr int RW = OUT_ROWS / (OUT_THREADS / 64);  // rows per wave
+  typename E::Raw uv[RW];
+  float gate[RW];
+#pragma unroll
+  for (int r = 0; r < RW; ++r) {
+    const int d = min(v0 + wave * RW + r, s.vdim - 1);
+    uv[r] = E::cached((const T *)a.uv.w + (size_t)(h * s.vdim + d) * ld + min(lane * 8, ld - 8));
+    gate[r] = a.g_off >= 0 ? a.proj[(size_t)tok * a.proj_ld + a.g_off + h * s.vdim + d] : 0.0f;
+  }
   if (wave == 0) {
     const float sink = a.sinks ? a.sinks[h] : 0.0f;
     float m = s.sink ? sink : -__builtin_inff(), z = 0.0f;
-    for (int k = lane; k < w.parts; k += 64) m = fmaxf(m, w.m[(row + k) * s.heads + h]);
+    for (int k = lane; k < w.parts; k += 64) {
+      const float mk = w.m[(row + k) * s.heads + h];
+      den[k] = w.z[(row + k) * s.heads + h];
+      weight[k] = mk;
+      m = fmaxf(m, mk);
+    }
     m = kxw::wave_max_f32(m);
     for (int k = lane; k < w.parts; k += 64) {
-      const float y = kx_expf(w.m[(row + k) * s.heads + h] - m);
-      weight[k] = y;
-      z = __builtin_fmaf(w.z[(row + k) * s.heads + h], y, z);
+      const float e = kx_expf(weight[k] - m);
+      weight[k] = e;
+      z = __builtin_fmaf(den[k], e, z);
     }
     const float inv = 1.0f / (kxr::wave_sum(z) + (s.sink ? kx_expf(sink - m) : 0.0f));
     for (int k = lane; k < w.parts; k += 64) weight[k] *= inv;
   }
   __syncthreads();
-  for (int c = tid; c < ld; c += 256) {
-    float v = 0.0f;
-    if (c < s.kv_rank) {
-#pragma unroll 8
-      for (int k = 0; k < w.parts; ++k) {  // a part without keys has not written its sums
-        const float x = w.o[((row + k) * s.heads + h) * vp + c];
-        v = weight[k] > 0.0f ? __builtin_fmaf(x, weight[k], v) : v;
+  for (int x = tq; x < quads; x += per) {
+    f32x4 v = {0.0f, 0.0f, 0.0f, 0.0f};
+    for (int k0 = share; k0 < w.parts; k0 += OUT_AHEAD * shares) {
+      if (x != tq || k0 != share)
+#pragma unroll
+        for (int j = 0; j < OUT_AHEAD; ++j) y[j] = part(k0 + j * shares, x);
+#pragma unroll
+      for (int j = 0; j < OUT_AHEAD; ++j) {
+        const int k = k0 + j * shares;
+        const float wt = k < w.parts ? weight[k] : 0.0f;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = wt > 0.0f ? __builtin_fmaf(y[j][e], wt, v[e]) : v[e];  // a part without keys has not written its sums
       }
     }
+    *(f32x4 *)(sum + share * ld + 4 * x) = v;
+  }
+  __syncthreads();
+  for (int c = tid; c < ld; c += OUT_THREADS) {
+    float v = 0.0f;
+    if (c < s.kv_rank)
+      for (int j = 0; j < shares; ++j) v += sum[j * ld + c];
     lat[c] = v;
   }
   __syncthreads();
-  constexpr int RW = OUT_ROWS / 4;  // rows per wave
   float acc[RW] = {};
   for (int x = lane * 8; x < ld; x += 512) {
     float l[8];
@@ -138,7 +332,8 @@ __global__ void __launch_bounds__(256) latent_out_k(KxLatentArgs a, KxWindowPart
 #pragma unroll
     for (int r = 0; r < RW; ++r) {
       float f[8];
-      E::unpack(f, E::cached((const T *)a.uv.w + (size_t)(h * s.vdim + min(v0 + wave * RW + r, s.vdim - 1)) * ld + x));
+      if (x >= 512) uv[r] = E::cached((const T *)a.uv.w + (size_t)(h * s.vdim + min(v0 + wave * RW + r, s.vdim - 1)) * ld + x);
+      E::unpack(f, uv[r]);
 #pragma unroll
       for (int e = 0; e < 8; ++e) acc[r] = __builtin_fmaf(f[e], l[e], acc[r]);
     }
@@ -147,8 +342,8 @@ __global__ void __launch_bounds__(256) latent_out_k(KxLatentArgs a, KxWindowPart
 #pragma unroll
   for (int r = 0; r < RW; ++r) {
     const int d = v0 + wave * RW + r;
-    const float y = kxr::wave_sum(acc[r]);
-    if (lane == 0 && d < s.vdim) out[d] = E::make(y * (a.g_off >= 0 ? kx_sigmoidf(a.proj[(size_t)tok * a.proj_ld + a.g_off + h * s.vdim + d]) : 1.0f));
+    const float o = kxr::wave_sum(acc[r]);
+    if (lane == 0 && d < s.vdim) out[d] = E::make(a.g_off >= 0 ? o * kx_sigmoidf(gate[r]) : o);
   }
 }
 
@@ -182,31 +377,62 @@ __global__ void __launch_bounds__(256) share_k(KxLatentArgs a, int n, int cap, i
   }
 }
 
+// LDS of latent_part_k without its tile, and keys of the tile that fits beside it
+template <class T>
+size_t part_lds(int row) { return (size_t)GROUP * (row + 8) * sizeof(T) + (GROUP * KEYS + 2 * GROUP) * 4; }
+template <class T>
+int part_keys(const KxLatentSpec &s) {
+  int keys = KEYS;
+  while (keys > 16 && (size_t)keys * kx_latent_row(s) * sizeof(T) + part_lds<T>(window_row(s)) > PART_LDS) keys >>= 1;  // 16: as the matrix cores take them
+  return keys;
+}
+// Parts of a step whose last token sees `total` keys: whole tiles, and no more workgroups than run at once as long as a
+// part has few tiles.
+template <class T>
+void plan_parts(const KxLatentSpec &s, int total, int tokens, Parts &p) {
+  p.keys = part_keys<T>(s);
+  const int tiles = kx_cdiv(total, p.keys), at_once = std::max(1, 2 * kx_device_cus());
+  p.per = std::max(1, (int)((long)tiles * kx_cdiv(s.heads, GROUP) * tokens / at_once));
+  p.parts = kx_cdiv(tiles, p.per);
+  while (p.parts > MAX_PARTS) p.parts = kx_cdiv(tiles, ++p.per);
+}
+size_t part_room(const KxLatentSpec &s) { return (size_t)s.heads * (kx_pad(s.kv_rank, 32) + 2); }
+
+template <class T, int NC>
+int parts_launch(const KxLatentArgs &a, const Parts &p, int tok0, int row, int vp, hipStream_t st) {
+  static std::atomic<bool> attr{false};
+  if (!attr) {
+    KX_HIP(hipFuncSetAttribute((const void *)latent_part_k<T, NC>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)MOST_LDS));
+    attr = true;
+  }
+  const size_t lds = (size_t)p.keys * kx_latent_row(a.s) * sizeof(T) + part_lds<T>(row);
+  KX_REQUIRE(lds <= MOST_LDS, "latent attention: cached rows of %d columns do not fit a workgroup", kx_latent_row(a.s));
+  hipLaunchKernelGGL((latent_part_k<T, NC>), dim3(p.parts, kx_cdiv(a.s.heads, GROUP), p.n), dim3(256), lds, st, a, p, tok0, row, vp);
+  KX_LAUNCH_CHECK();
+  return KX_OK;
+}
+
 template <class T>
 int few(const KxLatentArgs &a, hipStream_t st) {
   const KxLatentSpec &s = a.s;
-  const int tokens = a.batch * a.positions, row = window_row(s);
+  const int tokens = a.batch * a.positions, row = window_row(s), vp = kx_pad(s.kv_rank, 32);
   KX_REQUIRE(tokens <= a.x.q_tokens, "latent attention: %d tokens, room for %d", tokens, a.x.q_tokens);
   hipLaunchKernelGGL(absorb_k<T>, dim3(s.heads * kx_cdiv(s.kv_rank, ABS_COLS) + 1, tokens), dim3(256), (size_t)s.dim * 4, st, a, row);
   KX_LAUNCH_CHECK();
-  KxWindowArgs w;
-  w.s.heads = s.heads; w.s.dim = s.kv_rank + s.rot_dim; w.s.vdim = s.kv_rank; w.s.scale = s.scale; w.s.sink = s.sink;
-  int group = std::min(HEAD_GROUP, s.heads);
-  while (s.heads % group) --group;
-  w.s.kv_heads = s.heads / group;
-  w.c.k = w.c.v = a.rows; w.c.cap = a.cap; w.c.dp = row; w.c.vp = kx_pad(s.kv_rank, 32);
-  w.c.k_ld = w.c.v_ld = kx_latent_row(s);
-  w.c.shared = true;
-  w.q_f32 = a.x.q;
-  w.batch = a.batch; w.positions = a.positions; w.pos = a.pos;
-  w.part = a.x.part; w.part_floats = a.x.part_floats;
-  KxWindowParts p;
+  Parts p;
   for (int t0 = 0; t0 < tokens; t0 += p.n) {
-    int rc = kx_window_parts_launch(sizeof(T) == 4, w, t0, tokens - t0, &p, st);
+    plan_parts<T>(s, a.pos + a.positions, tokens - t0, p);
+    const size_t per_token = p.parts * part_room(s);
+    KX_REQUIRE(per_token <= a.x.part_floats, "latent attention: %zu floats of partials, room for %zu", per_token, a.x.part_floats);
+    p.n = (int)std::min<size_t>({(size_t)(tokens - t0), a.x.part_floats / per_token, (size_t)65535});
+    p.o = a.x.part;
+    p.m = p.o + (size_t)p.n * p.parts * s.heads * vp;
+    p.z = p.m + (size_t)p.n * p.parts * s.heads;
+    int rc = vp <= 512 ? parts_launch<T, 1>(a, p, t0, row, vp, st) : vp <= 1024 ? parts_launch<T, 2>(a, p, t0, row, vp, st) : parts_launch<T, 4>(a, p, t0, row, vp, st);
     if (rc) return rc;
-    const size_t lds = ((size_t)a.uv.ld + p.parts) * 4;
+    const size_t lds = ((size_t)5 * a.uv.ld + 2 * p.parts) * 4;
     KX_REQUIRE(lds <= 64 * 1024, "latent attention: %d parts of %d columns", p.parts, s.kv_rank);
-    hipLaunchKernelGGL(latent_out_k<T>, dim3(s.heads * kx_cdiv(s.vdim, OUT_ROWS), p.n), dim3(256), lds, st, a, p, t0, w.c.vp);
+    hipLaunchKernelGGL(latent_out_k<T>, dim3(s.heads * kx_cdiv(s.vdim, OUT_ROWS), p.n), dim3(OUT_THREADS), lds, st, a, p, t0, vp);
     KX_LAUNCH_CHECK();
   }
   return KX_OK;
@@ -280,11 +506,10 @@ void kx_latent_scratch(const KxLatentSpec &s, int max_batch, int max_context, in
   const size_t rows = (size_t)max_batch * s.heads * kx_pad(max_context, 64);
   x->k_elems = std::min(rows * kx_pad(s.dim + s.rot_dim, 32), EXPAND_BYTES / 2);
   x->v_elems = std::min(rows * kx_pad(s.vdim, 32), EXPAND_BYTES / 2);
-  KxWindowSpec few, many;  // partials: of all heads against the latent, and of every head against its own keys
-  few.heads = many.heads = many.kv_heads = s.heads; few.kv_heads = 1;
-  few.vdim = s.kv_rank; many.vdim = s.vdim;
-  x->part_floats = std::max(kx_window_part_floats(few, max_context, std::min(x->q_tokens, 64)),
-                            kx_window_part_floats(many, max_context, std::min(std::max(max_batch, step_tokens), 64)));
+  KxWindowSpec own;  // partials: of all heads against the latent , and of every head against its own keys
+  own.heads = own.kv_heads = s.heads; own.vdim = s.vdim;
+  const size_t parts = std::min(kx_cdiv(max_context, 8), MAX_PARTS);
+  x->part_floats = std::max(parts * part_room(s) * std::min(x->q_tokens, 4), kx_window_part_floats(own, max_context, std::min(std::max(max_batch, step_tokens), 64)));
 }
 
 void kx_latent_turns(const KxLatentSpec &s, int positions, float *out) {

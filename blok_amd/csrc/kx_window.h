@@ -21,10 +21,6 @@ struct KxWindowCache {
   void *k = nullptr, *v = nullptr;    // [batch][kv_heads][cap][dp], [..][vp]
   void *pk = nullptr, *pv = nullptr;  // [batch][kv_heads][blocks][dp], [..][vp]
   int cap = 0, blocks = 0, dp = 0, vp = 0;
-  // One token's attention (kx_window_parts_launch) also reads keys and values of one row in memory: rows of k_ld and v_ld
-  // elements (0: dp, vp), and with `shared` one set of rows for all key/value heads.
-  int k_ld = 0, v_ld = 0;
-  bool shared = false;
 };
 // Shape of the cache for sequences of up to max_context positions and steps of up to max_positions of them; the
 // element counts of one of k, v, pk, pv per sequence go to elems[4].
@@ -42,7 +38,6 @@ struct KxWindowArgs {
   void *out = nullptr;                    // [tokens][out_ld] of the model's type: heads * vdim, gated
   int out_ld = 0;
   void *q = nullptr;        // scratch [tokens][heads][dp] of the model's type
-  const float *q_f32 = nullptr;  // kx_window_parts_launch: the queries in 32-bit instead
   float *part = nullptr;    // scratch of part_floats floats (kx_window_part_floats)
   size_t part_floats = 0;
 };
@@ -51,10 +46,3 @@ size_t kx_window_part_floats(const KxWindowSpec &s, int max_context, int tokens)
 int kx_window_launch(bool f32, const KxWindowArgs &a, hipStream_t st);
 // The attention alone, with a.q and the cache's rows in place.
 int kx_window_attend(bool f32, const KxWindowArgs &a, hipStream_t st);
-// Tokens [tok0, tok0 + n) against parts of their keys, unmerged: [n][parts][heads * vp] sums, [n][parts][heads] maxima and as
-// many denominators.  n: as many of `tokens` as a.part has room for.
-struct KxWindowParts {
-  int n = 0, parts = 0;
-  const float *o = nullptr, *m = nullptr, *z = nullptr;
-};
-int kx_window_parts_launch(bool f32, const KxWindowArgs &a, int tok0, int tokens, KxWindowParts *out, hipStream_t st);

@@ -115,9 +115,8 @@ __global__ void __launch_bounds__(PART_THREADS) win_partial_k(KxWindowArgs a, in
   float *qv = win_lds;                 // [R][dp]
   float *sc = qv + R * c.dp;           // [R][ch]
   float *sum = sc + R * ch;            // [groups][RB][vp]
-  const size_t head = c.shared ? b : (size_t)b * s.kv_heads + g;
-  const int kld = c.k_ld ? c.k_ld : c.dp, vld = c.v_ld ? c.v_ld : c.vp;
-  const T *kc = (const T *)c.k + head * c.cap * kld, *vc = (const T *)c.v + head * c.cap * vld;
+  const size_t head = (size_t)b * s.kv_heads + g;
+  const T *kc = (const T *)c.k + head * c.cap * c.dp, *vc = (const T *)c.v + head * c.cap * c.vp;
   const T *pkc = (const T *)c.pk + head * c.blocks * c.dp, *pvc = (const T *)c.pv + head * c.blocks * c.vp;
   if (FUSED) {
     const float *pr = a.proj + (size_t)tok * a.proj_ld;
@@ -149,11 +148,8 @@ __global__ void __launch_bounds__(PART_THREADS) win_partial_k(KxWindowArgs a, in
       if (s.pool > 0 && (p + 1) % s.pool == 0 && p / s.pool < c.blocks) pool_block<T>(a, head, p / s.pool, tid, PART_THREADS);
     }
   } else {
-    const size_t q0 = ((size_t)tok * s.heads + g * R) * c.dp;
-    if (a.q_f32)
-      for (int x = tid; x < R * c.dp; x += PART_THREADS) qv[x] = a.q_f32[q0 + x];
-    else
-      for (int x = tid; x < R * c.dp; x += PART_THREADS) qv[x] = E::load((const T *)a.q + q0 + x);
+    const T *q = (const T *)a.q + ((size_t)tok * s.heads + g * R) * c.dp;
+    for (int x = tid; x < R * c.dp; x += PART_THREADS) qv[x] = E::load(q + x);
   }
   __syncthreads();
   const int base = p / c.cap * c.cap;  // position j of the window: slot j - base, one ring length more below it
@@ -165,7 +161,7 @@ __global__ void __launch_bounds__(PART_THREADS) win_partial_k(KxWindowArgs a, in
   const int l8 = lane & 7;
   for (int k0 = wave * 8; k0 < n; k0 += 32) {
     const int e = e0 + min(k0 + (lane >> 3), n - 1);
-    const T *key = e < nb ? pkc + (size_t)e * c.dp : kc + (size_t)slot_of(e) * kld;
+    const T *key = e < nb ? pkc + (size_t)e * c.dp : kc + (size_t)slot_of(e) * c.dp;
     for (int r0 = 0; r0 < R; r0 += RB) {
       float d[RB] = {};
       for (int x = l8 * 8; x < c.dp; x += 64) {
@@ -215,7 +211,7 @@ __global__ void __launch_bounds__(PART_THREADS) win_partial_k(KxWindowArgs a, in
       for (int k = grp; k < n; k += groups) {
         const int e = e0 + k;
         float vf[8];
-        E::unpack(vf, E::cached((e < nb ? pvc + (size_t)e * c.vp : vc + (size_t)slot_of(e) * vld) + col));
+        E::unpack(vf, E::cached((e < nb ? pvc + (size_t)e * c.vp : vc + (size_t)slot_of(e) * c.vp) + col));
 #pragma unroll
         for (int r = 0; r < RB; ++r) {
           const float w = sc[min(r0 + r, R - 1) * ch + k];
@@ -506,13 +502,15 @@ int check(const KxWindowArgs &a) {
   return KX_OK;
 }
 
+// parts and merge
 template <class T>
-int parts_launch(const KxWindowArgs &a, bool fused, int tok0, int tokens, KxWindowParts &out, hipStream_t st) {
+int attend_parts(const KxWindowArgs &a, bool fused, hipStream_t st) {
   const KxWindowSpec &s = a.s;
-  const int R = s.heads / s.kv_heads, total = most_keys(s, a.pos + a.positions), ch = part_keys(s, total, tokens), parts = kx_cdiv(total, ch);
+  const int tokens = a.batch * a.positions, R = s.heads / s.kv_heads;
+  const int total = most_keys(s, a.pos + a.positions), ch = part_keys(s, total, tokens), parts = kx_cdiv(total, ch);
   const size_t per_token = (size_t)parts * floats_per_part(s);
   KX_REQUIRE(per_token <= a.part_floats, "window attention: %zu floats of partials, room for %zu", per_token, a.part_floats);
-  const int n = (int)std::min<size_t>({(size_t)tokens, a.part_floats / per_token, (size_t)65535});
+  const int at_once = (int)std::min<size_t>({(size_t)tokens, a.part_floats / per_token, (size_t)65535});
   const size_t lds = ((size_t)R * a.c.dp + (size_t)R * ch + (size_t)(PART_THREADS / (a.c.vp / 8)) * RB * a.c.vp) * 4;
   KX_REQUIRE(lds <= 160 * 1024 - 256, "window attention: %d query heads of %d per key head do not fit a workgroup", R, s.dim);
   static std::atomic<bool> attr{false};
@@ -521,24 +519,14 @@ int parts_launch(const KxWindowArgs &a, bool fused, int tok0, int tokens, KxWind
     KX_HIP(hipFuncSetAttribute((const void *)win_partial_k<T, false>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 256));
     attr = true;
   }
-  float *po = a.part, *pm = po + (size_t)n * parts * s.heads * a.c.vp, *pz = pm + (size_t)n * parts * s.heads;
-  const dim3 grid(parts, s.kv_heads, n);
-  if (fused) hipLaunchKernelGGL((win_partial_k<T, true>), grid, dim3(PART_THREADS), lds, st, a, tok0, ch, po, pm, pz);
-  else hipLaunchKernelGGL((win_partial_k<T, false>), grid, dim3(PART_THREADS), lds, st, a, tok0, ch, po, pm, pz);
-  KX_LAUNCH_CHECK();
-  out.n = n; out.parts = parts; out.o = po; out.m = pm; out.z = pz;
-  return KX_OK;
-}
-
-// parts and merge
-template <class T>
-int attend_parts(const KxWindowArgs &a, bool fused, hipStream_t st) {
-  const int tokens = a.batch * a.positions;
-  KxWindowParts p;
-  for (int t0 = 0; t0 < tokens; t0 += p.n) {
-    int rc = parts_launch<T>(a, fused, t0, tokens - t0, p, st);
-    if (rc) return rc;
-    hipLaunchKernelGGL((win_merge_k<T>), dim3(a.s.heads, p.n), dim3(MERGE_THREADS), (size_t)p.parts * 4, st, a, t0, p.parts, p.o, p.m, p.z);
+  for (int t0 = 0; t0 < tokens; t0 += at_once) {
+    const int n = std::min(at_once, tokens - t0);
+    float *po = a.part, *pm = po + (size_t)n * parts * s.heads * a.c.vp, *pz = pm + (size_t)n * parts * s.heads;
+    const dim3 grid(parts, s.kv_heads, n);
+    if (fused) hipLaunchKernelGGL((win_partial_k<T, true>), grid, dim3(PART_THREADS), lds, st, a, t0, ch, po, pm, pz);
+    else hipLaunchKernelGGL((win_partial_k<T, false>), grid, dim3(PART_THREADS), lds, st, a, t0, ch, po, pm, pz);
+    KX_LAUNCH_CHECK();
+    hipLaunchKernelGGL((win_merge_k<T>), dim3(s.heads, n), dim3(MERGE_THREADS), (size_t)parts * 4, st, a, t0, parts, po, pm, pz);
     KX_LAUNCH_CHECK();
   }
   return KX_OK;
@@ -598,8 +586,4 @@ int kx_window_launch(bool f32, const KxWindowArgs &a, hipStream_t st) { return f
 int kx_window_attend(bool f32, const KxWindowArgs &a, hipStream_t st) {
   const int rc = check(a);
   return rc ? rc : f32 ? attend<float>(a, st) : attend<uint16_t>(a, st);
-}
-int kx_window_parts_launch(bool f32, const KxWindowArgs &a, int tok0, int tokens, KxWindowParts *out, hipStream_t st) {
-  const int rc = check(a);
-  return rc ? rc : f32 ? parts_launch<float>(a, false, tok0, tokens, *out, st) : parts_launch<uint16_t>(a, false, tok0, tokens, *out, st);
 }
