@@ -23,6 +23,22 @@ int kx_expert_route_launch(bool f32, KxExpertArgs &e, const KxExpertSlots &s, in
 // x[t] += sum_j y[slot of choice j of t], f32 rows of `width`
 int kx_expert_combine_launch(const KxExpertSlots &s, const float *y, float *x, int tokens, int top, int width, hipStream_t st);
 
+// A feed-forward of experts beside another product that is added to the same residual rows:
+//   x_t <- x_t + out.m row_t + sum_j weight_j down[id_j] glu(gu[id_j] h_t)
+struct KxExpertFf {
+  KxLinArgs gu, out;          // the first expert's (gate, up) with the rows h in front (one norm of x); the other product
+  KxMat down;                 // the first expert's
+  size_t gu_stride = 0, down_stride = 0;  // elements from one expert's matrix to the next
+  KxExpertArgs e;             // experts, top, logits, logits_ld, bias
+  KxExpertSlots s;
+  const void *h = nullptr;    // the rows h, if they are in memory, rows of gu.m.ld elements; nullptr: built where they are needed
+  void *h_buf = nullptr, *row_buf = nullptr;  // room for them and for the other product's rows
+  void *mid = nullptr;        // [tokens * top][down.ld] of the model's type
+  float *y = nullptr;         // f32 [tokens * top][width]
+};
+// Up to KX_GEMV_TOKENS tokens two launches where the sizes allow; otherwise sorted by expert.
+int kx_expert_ff_launch(bool f32, const KxExpertFf &f, int tokens, hipStream_t st);
+
 namespace kxe {
 
 // The `top` largest of logits + bias, the lower index first where two are equal, and the softmax over them.  One wave.

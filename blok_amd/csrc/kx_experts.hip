@@ -76,3 +76,38 @@ int kx_expert_combine_launch(const KxExpertSlots &s, const float *y, float *x, i
   KX_LAUNCH_CHECK();
   return KX_OK;
 }
+
+int kx_expert_ff_launch(bool f32, const KxExpertFf &f, int tokens, hipStream_t st) {
+  KxLinArgs gu = f.gu;
+  gu.epi = KX_LIN_GLU;
+  gu.mid = f.mid;
+  gu.mid_ld = f.down.ld;
+  KxExpertArgs e = f.e, eo = f.e;
+  e.ids = eo.ids = f.s.ids;
+  e.weights = eo.weights = f.s.weights;
+  e.stride = f.gu_stride;
+  eo.stride = f.down_stride; eo.w = f.down.w; eo.ld = f.down.ld; eo.mid = f.mid; eo.mid_ld = f.down.ld;
+  if (kx_expert_small(f32, gu, f.out, eo, tokens)) {
+    KX_DO(kx_expert_in_launch(f32, gu, e, st));
+    return kx_expert_out_launch(f32, f.out, eo, st);
+  }
+  const void *h = f.h;
+  if (!h) {
+    KX_DO(kx_rows_launch(f32, gu.row, tokens, f.h_buf, gu.m.ld, st));
+    h = f.h_buf;
+  }
+  KX_DO(kx_expert_route_launch(f32, e, f.s, tokens, st));
+  e.gather = f.s.gather;
+  KX_DO(kx_expert_gemm_launch(f32, gu, e, h, gu.m.ld, st));
+  KX_DO(kx_linear_launch(f32, f.out, f.row_buf, st));
+  KxLinArgs down;
+  down.m = f.down;
+  down.tokens = tokens;
+  down.row.cols = f.down.cols;
+  down.out = f.y;
+  down.out_ld = f.down.rows;
+  e.gather = nullptr;
+  e.stride = f.down_stride;
+  KX_DO(kx_expert_gemm_launch(f32, down, e, f.mid, f.down.ld, st));
+  return kx_expert_combine_launch(f.s, f.y, f.out.streams, tokens, e.top, f.down.rows, st);
+}

@@ -641,39 +641,16 @@ int HybridModel::step(const uint32_t *d_ids, bool sample, int C) {
       KX_DO(latent(l, w, C));
     }
     if (experts) {
-      KxLinArgs gu;
-      KxExpertArgs e, eo;
-      read(gu, w.gu, w.norm1, w.hc[0]);
-      gu.epi = KX_LIN_GLU;
-      gu.mid = mid; gu.mid_ld = w.down.ld; gu.limit = l.limit; gu.alpha = l.alpha; gu.bias = l.bias;
-      e.experts = l.experts; e.top = l.top;
-      e.logits = proj + w.router_off; e.logits_ld = proj_ld; e.bias = w.router_b;
-      e.ids = slots_of.ids; e.weights = slots_of.weights;
-      eo = e;
-      e.stride = w.gu_stride;
-      eo.stride = w.down_stride; eo.w = w.down.w; eo.ld = w.down.ld; eo.mid = mid; eo.mid_ld = w.down.ld;
-      if (kx_expert_small(f32, gu, out, eo, T)) {
-        KX_DO(kx_expert_in_launch(f32, gu, e, st));
-        KX_DO(kx_expert_out_launch(f32, out, eo, st));
-      } else {
-        const char *h = (const char *)rows;  // the first product has built them
-        if (T <= KX_GEMV_TOKENS) KX_DO(kx_rows_launch(f32, gu.row, T, rows, w.gu.ld, st));
-        else if (shifted) h += (size_t)in.row.n_mix * T * w.in.ld * es;
-        KX_DO(kx_expert_route_launch(f32, e, slots_of, T, st));
-        e.gather = slots_of.gather;
-        KX_DO(kx_expert_gemm_launch(f32, gu, e, h, w.gu.ld, st));
-        KX_DO(kx_linear_launch(f32, out, out_rows, st));
-        KxLinArgs down;
-        down.m = w.down;
-        down.tokens = T;
-        down.row.cols = w.down.cols;
-        down.out = expert_y;
-        down.out_ld = W;
-        e.gather = nullptr;
-        e.stride = w.down_stride;
-        KX_DO(kx_expert_gemm_launch(f32, down, e, mid, w.down.ld, st));
-        KX_DO(kx_expert_combine_launch(slots_of, expert_y, streams, T, l.top, W, st));
-      }
+      KxExpertFf f;
+      read(f.gu, w.gu, w.norm1, w.hc[0]);
+      f.gu.limit = l.limit; f.gu.alpha = l.alpha; f.gu.bias = l.bias;
+      f.out = out;
+      f.down = w.down; f.gu_stride = w.gu_stride; f.down_stride = w.down_stride;
+      f.e.experts = l.experts; f.e.top = l.top; f.e.logits = proj + w.router_off; f.e.logits_ld = proj_ld; f.e.bias = w.router_b;
+      f.s = slots_of;
+      if (T > KX_GEMV_TOKENS) f.h = (const char *)rows + (shifted ? (size_t)in.row.n_mix * T * w.in.ld * es : 0);  // the first product has built them
+      f.h_buf = rows; f.row_buf = out_rows; f.mid = mid; f.y = expert_y;
+      KX_DO(kx_expert_ff_launch(f32, f, T, st));
     } else {
       KX_DO(kx_linear_launch(f32, out, out_rows, st));
     }

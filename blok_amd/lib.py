@@ -63,7 +63,26 @@ class KxLinearArgs(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("f32", "tokens", "rows", "cols", "ld", "row_kind", "epilogue", "streams", "groups", "heads",
                                          "vdim", "x_ld", "gate_ld", "out_ld")] + [
         (n, C.c_float) for n in ("eps", "limit", "alpha", "bias")] + [
-        (n, C.c_void_p) for n in ("d_w", "d_x", "d_streams_in", "d_in", "d_norm", "d_o", "d_gate", "d_mix", "d_outw", "d_out")]
+        (n, C.c_void_p) for n in ("d_w", "d_x", "d_streams_in", "d_in", "d_norm", "d_o", "d_gate", "d_mix", "d_outw", "d_out")] + [
+        (n, C.c_int32) for n in ("w_per_column", "gate_first", "head_ld", "tail_ld", "n_mix", "batch", "streams_ld", "act_rows", "mid_ld", "head_dim")] + [
+        ("var_row", C.c_int32 * 8), ("head_stride", C.c_int64)] + [(n, C.c_void_p) for n in ("d_tail", "d_mu", "d_prev", "d_prev_out", "d_mid")]
+
+
+class KxSsdConfig(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("heads", "vdim", "state", "groups", "taps")]
+
+
+class KxWkvConfig(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("heads", "dim", "rank")]
+
+
+class KxLatentConfig(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("heads", "dim", "rot_dim", "rot", "vdim", "kv_rank", "sink", "gate", "no_expand")] + [
+        ("scale", C.c_float), ("eps", C.c_float), ("base", C.c_double)]
+
+
+class KxExpertsConfig(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("width", "ff", "experts", "top", "cols")] + [(n, C.c_float) for n in ("limit", "alpha", "bias")]
 
 
 DTYPES = {"bfloat16": 0, "float32": 1}
@@ -142,6 +161,20 @@ _SIGS = {
     "kx_delta_destroy": [_P],
     "kx_delta_restart": [_P, _P],
     "kx_delta_run": [_P, _P, _I, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _P, _P],
+    "kx_ssd_create": [C.POINTER(KxSsdConfig), _I, _I, _PP],
+    "kx_ssd_destroy": [_P],
+    "kx_ssd_restart": [_P, _P],
+    "kx_ssd_run": [_P, _P, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _P, _P],
+    "kx_wkv_create": [C.POINTER(KxWkvConfig), C.c_int, _I, _I, _PP],
+    "kx_wkv_destroy": [_P],
+    "kx_wkv_restart": [_P, _P],
+    "kx_wkv_run": [_P, _P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _P, _P],
+    "kx_latent_create": [C.POINTER(KxLatentConfig), C.c_int, _I, _I, _I, _PP],
+    "kx_latent_destroy": [_P],
+    "kx_latent_run": [_P, _P, _I, _P, _I, _I, _I, _P, _P, _P, _P, _I, _I, _I, _P, _I, _P],
+    "kx_experts_create": [C.POINTER(KxExpertsConfig), C.c_int, _I, _PP],
+    "kx_experts_destroy": [_P],
+    "kx_experts_run": [_P, _P, _P, _F, _P, _P, _P, _P, _P, _P, _I, _P, _P],
     "kx_linear_run": [C.POINTER(KxLinearArgs), _P, _P],
     "kx_open_options_default": [C.POINTER(KxOpenOptions)],
     "kx_model_open": [C.c_char_p, C.POINTER(KxOpenOptions), _PP],

@@ -280,11 +280,35 @@ int kx_generate(kx_model *model, const uint32_t *h_prompt, int32_t batch, int32_
  * kx_delta_*: the gated delta rule behind short causal convolutions with silu.  d_proj f32 [tokens][proj_ld] holds q, k
  *   [kv_heads][dim], v [heads][vdim] and the projections of step size and decay, b and a [heads].  d_conv f32 [channels][taps]
  *   (q, k, v channels in turn); d_o f32 [tokens][heads * vdim].  A kx_delta holds state and convolution inputs.
- * kx_linear_run: y = W row with the row built from residual streams (row_kind 1: w * groupnorm(sum_s in[s] x_s)), from the
- *   delta rule's read-out (row_kind 2: per head rms norm * w * silu(gate)) or taken from memory (0), and the product stored
- *   (epilogue 0), made into a clamped gated activation (1; W's rows are blocks of 32 gate rows and their 32 up rows), or
- *   written to all streams (2: x_t <- sum_s mix[s][t] x_s + outw[t] y).  Matrices have rows of `ld` elements, a multiple of
- *   64, zero beyond `cols`; rows in memory (x, mid) likewise.                                                            */
+ * kx_ssd_*: state-space duality (Mamba-2) behind a short causal convolution with silu.  d_proj f32 [tokens][proj_ld]: x
+ *   [heads][vdim], B [groups][state], C [groups][state] from x_off on, the step size's projection [heads] at dt_off.  Per head,
+ *   with dt = softplus(. + dt_bias): S <- exp(-exp(A_log) dt) S + dt B x^T, y = S^T C + skip x.  d_conv f32 [channels][taps],
+ *   d_conv_bias [channels] or NULL; d_y f32 [tokens][heads * vdim].  A kx_ssd holds state and convolution inputs.
+ * kx_wkv_*: linear recurrence with a decay per key channel and a bonus for the current token (RWKV time mixing).  d_proj f32
+ *   [tokens][proj_ld]: r, k, v [heads][dim] and the decay's low-rank projection [rank].  Per head, with w = exp(-exp(W2
+ *   tanh(.) + w0)): o = (S + diag(u) k v^T)^T r, S <- diag(w) S + k v^T.  d_w2 [heads * dim][rank] of the number format, rows of
+ *   `rank` padded to a multiple of 64; d_w0, d_u f32 [heads][dim]; d_o f32 [tokens][heads * dim].
+ * kx_latent_*: latent attention.  d_q f32 [tokens][q_ld]: per head dim unrotated and rot_dim to be rotated dimensions; d_proj f32
+ *   [tokens][proj_ld]: the latent [kv_rank] and the key part that the heads share [rot_dim] from kv_off on, with `gate` the
+ *   output gate's pre-activation [heads][vdim] at g_off.  The latent is RMS-normed with d_kv_norm; keys are d_uk
+ *   [heads * dim][kv_rank] times it, values d_uv [heads * vdim][kv_rank] (rows padded to a multiple of 64).  The first `rot` of
+ *   the rot_dim dimensions turn in pairs (d, d + rot / 2) by position * base^(-2 d / rot).  With `sink` the softmax's denominator
+ *   has exp(d_sinks[head]) more.  d_out [tokens][out_ld] of the number format.  A kx_latent holds the cache and scratch.
+ * kx_experts_*: x <- x + W row + sum over a token's `top` experts of weight * expert(h), h = rmsnorm(x) * d_norm, in place in
+ *   d_x f32 [tokens][width].  The experts are those with the largest d_router h + d_router_bias, the weights the softmax over the
+ *   chosen logits.  d_gu [experts][rows][ld of width]: blocks of 32 gate rows and their 32 up rows; activation as epilogue 1 of
+ *   kx_linear_run (silu: limit infinite, alpha 1, bias 0); d_down [experts][width][ld of ff].  d_w [width][ld of cols] and d_rows
+ *   [tokens][ld of cols] are the product beside them.  d_ids i32 [tokens][top] or NULL receives the choice.
+ * kx_linear_run: y = W row with the row built from residual streams (row_kind 1: w * groupnorm(sum_s in[s] x_s)), from a
+ *   recurrence's read-out (row_kind 2: per head rms norm * w * silu(gate); gate_first: the gate in front of the norm;
+ *   w_per_column: w [heads][vdim]; d_tail: the row goes on with elements of the number format from column head_ld on), as mixes
+ *   of a normed row h and the one of the position before it (row_kind 3: h + (h' - h) mu[m] for the matrix rows from
+ *   var_row[m] on, a multiple of 128, and h itself from var_row[n_mix] on; d_prev [batch][cols] is h' of the step's first
+ *   position, d_prev_out receives the last h), as tanh of f32 rows of streams_ld (row_kind 4), or taken from memory (0), and
+ *   the product stored (epilogue 0; the last act_rows rows of W go through gelu to d_mid instead), made into a clamped gated
+ *   activation (1; W's rows are blocks of 32 gate rows and their 32 up rows), written to all streams (2: x_t <- sum_s
+ *   mix[s][t] x_s + outw[t] y), or stored in the number format as a block per head (3: head h of token t at h * head_stride +
+ *   t * out_ld).  Matrices have rows of `ld` elements, a multiple of 64, zero beyond `cols`; rows in memory (x, mid) likewise. */
 typedef struct kx_window_config {
   int32_t heads, kv_heads, dim, vdim, size, pool, sink, gate;
   float scale, eps;
@@ -306,17 +330,60 @@ int kx_delta_restart(kx_delta *d, void *stream);
 int kx_delta_run(kx_delta *d, const void *d_proj, int32_t proj_ld, int32_t q_off, int32_t k_off, int32_t v_off, int32_t b_off,
                  int32_t a_off, const void *d_conv, const void *d_a_log, const void *d_dt_bias, int32_t batch, int32_t positions,
                  void *d_o, void *stream);
+typedef struct kx_ssd_config {
+  int32_t heads, vdim, state, groups, taps;
+} kx_ssd_config;
+typedef struct kx_ssd kx_ssd;
+int kx_ssd_create(const kx_ssd_config *cfg, int32_t max_batch, int32_t max_positions, kx_ssd **out);
+int kx_ssd_destroy(kx_ssd *d);
+int kx_ssd_restart(kx_ssd *d, void *stream);
+int kx_ssd_run(kx_ssd *d, const void *d_proj, int32_t proj_ld, int32_t x_off, int32_t dt_off, const void *d_conv, const void *d_conv_bias,
+               const void *d_a_log, const void *d_dt_bias, const void *d_skip, int32_t batch, int32_t positions, void *d_y, void *stream);
+typedef struct kx_wkv_config {
+  int32_t heads, dim, rank;
+} kx_wkv_config;
+typedef struct kx_wkv kx_wkv;
+int kx_wkv_create(const kx_wkv_config *cfg, int f32, int32_t max_batch, int32_t max_positions, kx_wkv **out);
+int kx_wkv_destroy(kx_wkv *d);
+int kx_wkv_restart(kx_wkv *d, void *stream);
+int kx_wkv_run(kx_wkv *d, const void *d_proj, int32_t proj_ld, int32_t r_off, int32_t k_off, int32_t v_off, int32_t w_off, const void *d_w2,
+               const void *d_w0, const void *d_u, int32_t batch, int32_t positions, void *d_o, void *stream);
+typedef struct kx_latent_config {
+  int32_t heads, dim, rot_dim, rot, vdim, kv_rank, sink, gate;
+  int32_t no_expand; /* long steps too attend to the cached rows themselves, as where a context's keys and values do not fit */
+  float scale, eps;
+  double base;
+} kx_latent_config;
+typedef struct kx_latent kx_latent;
+int kx_latent_create(const kx_latent_config *cfg, int f32, int32_t max_batch, int32_t max_context, int32_t max_positions, kx_latent **out);
+int kx_latent_destroy(kx_latent *d);
+int kx_latent_run(kx_latent *d, const void *d_q, int32_t q_ld, const void *d_proj, int32_t proj_ld, int32_t kv_off, int32_t g_off,
+                  const void *d_kv_norm, const void *d_uk, const void *d_uv, const void *d_sinks, int32_t batch, int32_t positions,
+                  int32_t pos, void *d_out, int32_t out_ld, void *stream);
+typedef struct kx_experts_config {
+  int32_t width, ff, experts, top, cols; /* cols: of the product beside the experts */
+  float limit, alpha, bias;
+} kx_experts_config;
+typedef struct kx_experts kx_experts;
+int kx_experts_create(const kx_experts_config *cfg, int f32, int32_t max_tokens, kx_experts **out);
+int kx_experts_destroy(kx_experts *d);
+int kx_experts_run(kx_experts *d, void *d_x, const void *d_norm, float eps, const void *d_router, const void *d_router_bias, const void *d_gu,
+                   const void *d_down, const void *d_w, const void *d_rows, int32_t tokens, void *d_ids, void *stream);
 typedef struct kx_linear_args {
   int32_t f32, tokens, rows, cols, ld, row_kind, epilogue, streams, groups, heads, vdim, x_ld, gate_ld, out_ld;
   float eps, limit, alpha, bias;
   const void *d_w, *d_x, *d_streams_in, *d_in, *d_norm, *d_o, *d_gate, *d_mix, *d_outw;
   void *d_out; /* epilogue 0: f32 [tokens][out_ld]; 1: [tokens][out_ld] of the format; 2: f32 [tokens][streams][rows], in place */
+  int32_t w_per_column, gate_first, head_ld, tail_ld, n_mix, batch, streams_ld, act_rows, mid_ld, head_dim, var_row[8];
+  int64_t head_stride;
+  const void *d_tail, *d_mu, *d_prev;
+  void *d_prev_out, *d_mid;
 } kx_linear_args;
-int kx_linear_run(const kx_linear_args *args, void *d_row_scratch, void *stream); /* scratch: tokens * ld elements of the format */
+int kx_linear_run(const kx_linear_args *args, void *d_row_scratch, void *stream); /* scratch: tokens * ld elements of the format per variant of the rows */
 /* ---- model directories ---------------------------------------------------------------------
  * kx_model_open  : reads <dir>/config.json, finds the design it names in the library's registry and opens the model
- *                  with it.  Two designs are known: Kimi-K2 (config.json of the checkpoint with runtime-index.blok
- *                  beside it; bfloat16) and Kagalorn (config.json and safetensors files; bfloat16 or float32).
+ *                  with it.  Three designs are known: Kimi-K2 (config.json of the checkpoint with runtime-index.blok
+ *                  beside it; bfloat16), Kagalorn and Rapitar (config.json and safetensors files; bfloat16 or float32).
  *                  Every kx_model entry point works on the result; those that set up a mechanism only Kimi-K2 has
  *                  (kx_model_set_fusion, _set_exact, _set_attention_kernel, routing, latent cache rows) return an error
  *                  on another design.
@@ -354,7 +421,7 @@ int kx_restart(kx_model *model, int32_t batch);
 int kx_extend(kx_model *model, const uint32_t *h_ids, int32_t n, const int32_t *h_want, int32_t n_want, float *h_logits);
 /* The residual stream (sum of the streams of a design that has several) after every layer, kept for every position
  * while the record is on: h_out f32 [n][batch][hidden] for positions pos0 .. pos0 + n - 1.  For parity checks;
- * Kagalorn only. */
+ * not for Kimi-K2. */
 int kx_model_set_residual_record(kx_model *model, int on);
 int kx_model_residual(kx_model *model, int32_t layer, int32_t pos0, int32_t n, float *h_out);
 /* ---- checkpoint: runtime-index.blok -> resident weights ----------------------------------------

@@ -163,11 +163,11 @@ def tokens(cfg, n, seed):
     return np.random.default_rng(seed).integers(0, cfg["vocab"], n)
 
 
-def greedy(cfg, w, prompt, n):
+def greedy(cfg, w, prompt, n, forward=K.forward):
     """Greedy continuation by the plain forward pass, whole sequence every time, and the smallest top-2 gap met."""
     ids, gap = list(map(int, prompt)), np.inf
     for _ in range(n):
-        row = K.forward(cfg, w, ids)[-1]
+        row = forward(cfg, w, ids)[-1]
         top = np.sort(row)[-2:]
         gap = min(gap, (top[1] - top[0]) / np.std(row))
         ids.append(int(np.argmax(row)))
