@@ -168,6 +168,11 @@ lin_gemv_k(KxLinArgs a, KxExpertArgs x) {
   int blk = blockIdx.x, c = 0;
   load(bufA, blk, 0);
   if (MODE == GV_EXPERT_OUT && (int)threadIdx.x < x.top) eid[threadIdx.x] = x.ids[tok0 * x.top + threadIdx.x];
+  uint32_t need = ~0u;  // variants that this workgroup's rows meet
+  if constexpr (MODE == GV_VARIANTS) {
+    need = 0;
+    for (int k = blockIdx.x; k < nblk; k += gridDim.x) need |= 1u << variant_of(a, 2 * k * GEMV_WAVES);
+  }
 #pragma unroll
   for (int t = 0; t < NT; ++t)
     if (t < tokens) {
@@ -181,7 +186,7 @@ lin_gemv_k(KxLinArgs a, KxExpertArgs x) {
           for (int y = threadIdx.x; y < el; y += GEMV_WAVES * 64) row[nc0 * CHUNK + j * el + y] = y < x.ld ? m[y] : E::make(0.0f);
         }
       }
-      kxr::build_row<T>(a.row, tok0 + t, row, ld, u, xl, blockIdx.x == 0);
+      kxr::build_row<T>(a.row, tok0 + t, row, ld, u, xl, blockIdx.x == 0, need);
     }
   float acc[2 * NT];
 #pragma unroll
@@ -241,10 +246,10 @@ lin_gemv_k(KxLinArgs a, KxExpertArgs x) {
   }
 }
 
-template <class T>
+template <class T, int KIND>
 __global__ void __launch_bounds__(256) row_k(KxRowArgs a, T *out, int ld) {
   extern __shared__ float row_lds[];
-  kxr::build_row<T>(a, blockIdx.x, out + (size_t)blockIdx.x * ld, ld, row_lds, (size_t)gridDim.x * ld, true);
+  kxr::build_row<T, KIND>(a, blockIdx.x, out + (size_t)blockIdx.x * ld, ld, row_lds, (size_t)gridDim.x * ld, true);
 }
 
 // ---- bf16 GEMM ----
@@ -450,18 +455,28 @@ int gemv_nt(const KxLinArgs &a, size_t lds, hipStream_t st) {
   return gemv_launch<T, NT, EPI, GV_PLAIN>(a, KxExpertArgs(), lds, 1, st);
 }
 
-template <class T>
-int rows_launch(const KxRowArgs &r, int tokens, T *out, int ld, hipStream_t st) {
+template <class T, int KIND>
+int rows_kind(const KxRowArgs &r, int tokens, T *out, int ld, hipStream_t st) {
   const size_t scratch = (size_t)kx_row_scratch(r) * 4;
   KX_REQUIRE(out && scratch <= 160 * 1024 - 1024, "kx_linear: rows of %d columns do not fit a workgroup", r.cols);
   static std::atomic<bool> attr{false};
   if (!attr) {
-    KX_HIP(hipFuncSetAttribute((const void *)row_k<T>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024));
+    KX_HIP(hipFuncSetAttribute((const void *)row_k<T, KIND>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024));
     attr = true;
   }
-  hipLaunchKernelGGL((row_k<T>), dim3(tokens), dim3(256), scratch, st, r, out, ld);
+  hipLaunchKernelGGL((row_k<T, KIND>), dim3(tokens), dim3(256), scratch, st, r, out, ld);
   KX_LAUNCH_CHECK();
   return KX_OK;
+}
+template <class T>
+int rows_launch(const KxRowArgs &r, int tokens, T *out, int ld, hipStream_t st) {
+  switch (r.kind) {
+    case KX_ROW_NORM: return rows_kind<T, KX_ROW_NORM>(r, tokens, out, ld, st);
+    case KX_ROW_GATED: return rows_kind<T, KX_ROW_GATED>(r, tokens, out, ld, st);
+    case KX_ROW_SHIFT: return rows_kind<T, KX_ROW_SHIFT>(r, tokens, out, ld, st);
+    case KX_ROW_TANH: return rows_kind<T, KX_ROW_TANH>(r, tokens, out, ld, st);
+  }
+  return rows_kind<T, KX_ROW_PLAIN>(r, tokens, out, ld, st);
 }
 
 // GEMM over rows in memory; GROUP: e.max_tiles tiles of slots

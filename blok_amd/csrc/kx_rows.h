@@ -100,13 +100,16 @@ __device__ __forceinline__ void group_scales(float *part, int groups, int spg, i
 }
 
 // Row `tok` into dst[0 .. ld), variants vstride apart.  u: LDS scratch of kx_row_scratch(a) floats.  Whole workgroup; ends
-// with a barrier.  keep: this workgroup writes what the row's kind carries over to the next step.
-template <class T>
-__device__ __forceinline__ void build_row(const KxRowArgs &a, int tok, T *dst, int ld, float *u, size_t vstride = 0, bool keep = false) {
-  const int tid = threadIdx.x, n = blockDim.x, lane = tid & 63, wave = tid >> 6, nw = n >> 6;
+// with a barrier.  keep: this workgroup writes what the row's kind carries over to the next step.  need: the variants
+// to build, a bit each.
+// KIND: the row's kind where it is known when the kernel is compiled.
+template <class T, int KIND = -1>
+__device__ __forceinline__ void build_row(const KxRowArgs &a, int tok, T *dst, int ld, float *u, size_t vstride = 0, bool keep = false,
+                                          uint32_t need = ~0u) {
+  const int tid = threadIdx.x, n = blockDim.x, lane = tid & 63, wave = tid >> 6, nw = n >> 6, kind = KIND >= 0 ? KIND : a.kind;
   if (a.rows_map) tok = a.rows_map[tok];
   const int xld = a.streams_ld ? a.streams_ld : a.n_streams * a.cols;
-  if (a.kind == KX_ROW_NORM) {
+  if (kind == KX_ROW_NORM) {
     float *part = u + a.cols;
     const float *x = a.streams + (size_t)tok * xld;
     const int gs = a.cols / a.groups, spg = max(1, nw / a.groups), units = a.groups * spg, per = (gs + spg - 1) / spg;
@@ -126,7 +129,7 @@ __device__ __forceinline__ void build_row(const KxRowArgs &a, int tok, T *dst, i
     __syncthreads();
     group_scales(part, a.groups, spg, gs, a.eps);
     for (int c = tid; c < ld; c += n) dst[c] = Elem<T>::make(c < a.cols ? u[c] * part[(c / gs) * spg] * a.w[c] : 0.0f);
-  } else if (a.kind == KX_ROW_SHIFT) {
+  } else if (kind == KX_ROW_SHIFT) {
     const bool first = tok < a.batch;
     const float *x = a.streams + (size_t)tok * xld, *x1 = first ? a.prev + (size_t)tok * a.cols : x - (size_t)a.batch * xld;
     float v = 0.0f, v1 = 0.0f;
@@ -144,10 +147,11 @@ __device__ __forceinline__ void build_row(const KxRowArgs &a, int tok, T *dst, i
         d = (first ? x1[c] : x1[c] * sc1 * w) - h;
         if (last) a.prev_out[(size_t)(tok + a.batch - a.tokens) * a.cols + c] = h;
       }
-      for (int m = 0; m < a.n_mix; ++m) dst[m * vstride + c] = Elem<T>::make(c < a.cols ? __builtin_fmaf(d, a.mu[(size_t)m * a.cols + c], h) : 0.0f);
+      for (int m = 0; m < a.n_mix; ++m)
+        if (need >> m & 1) dst[m * vstride + c] = Elem<T>::make(c < a.cols ? __builtin_fmaf(d, a.mu[(size_t)m * a.cols + c], h) : 0.0f);
       dst[a.n_mix * vstride + c] = Elem<T>::make(h);
     }
-  } else if (a.kind == KX_ROW_GATED) {
+  } else if (kind == KX_ROW_GATED) {
     const int cols = a.heads * a.vdim, hl = a.tail ? a.head_ld : ld;
     const float *o = a.o + (size_t)tok * cols, *gate = a.gate + (size_t)tok * a.gate_ld;
     auto gated = [&](int c) { return a.gate_first ? o[c] * gate[c] * sigmoid_for<T>(gate[c]) : o[c]; };
@@ -188,7 +192,7 @@ __device__ __forceinline__ void build_row(const KxRowArgs &a, int tok, T *dst, i
       const T *x = (const T *)a.tail + (size_t)tok * a.tail_ld;
       for (int c = tid * 8; c < ld - hl; c += n * 8) *(typename Elem<T>::Raw *)(dst + hl + c) = Elem<T>::cached(x + c);
     }
-  } else if (a.kind == KX_ROW_TANH) {
+  } else if (kind == KX_ROW_TANH) {
     const float *x = a.streams + (size_t)tok * xld;
     for (int c = tid; c < ld; c += n) dst[c] = Elem<T>::make(c < a.cols ? tanhf(x[c]) : 0.0f);
   } else {

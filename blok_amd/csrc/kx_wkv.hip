@@ -88,14 +88,22 @@ __host__ __device__ __forceinline__ Work work_of(const KxWkvArgs &a) {
   return w;
 }
 
-// one workgroup per (block, head): thread (j, s) goes through token j's channels s, s + 16, ...
+// One workgroup per (block, head): thread (j, s) goes through token j's channels s, s + 16, ...  Keys and decays have NB - 1 rows
+// of zeros in front, which the tokens before the block are.
+__host__ __device__ constexpr int coef_stride(int dim) { return dim + (dim < KX_SCAN_MAX_DIM ? 16 : 4); }
+constexpr size_t coef_lds(int dim) { return (size_t)(5 * NB - 2) * coef_stride(dim) * 4; }
 __global__ void __launch_bounds__(256) wkv_coef_k(KxWkvArgs a) {
   extern __shared__ float cf_lds[];
-  const int D = a.s.dim, STR = D + 16, tid = threadIdx.x, sl = tid & 15, j = tid >> 4;
+  const int D = a.s.dim, STR = coef_stride(D), tid = threadIdx.x, sl = tid & 15, j = tid >> 4;
   const int t0 = blockIdx.x * NB, h = blockIdx.y, b = blockIdx.z, padded = kx_scan_padded(a.positions);
   const Work w = work_of(a);
   const int HD = a.s.heads * D;
-  float *rs = cf_lds, *ks = rs + NB * STR, *ws = ks + NB * STR;
+  float *rs = cf_lds, *ks = rs + (2 * NB - 1) * STR, *ws = ks + (2 * NB - 1) * STR;  // row 0 is the block's first token
+  for (int x = tid; x < (NB - 1) * STR; x += 256) {
+    rs[NB * STR + x] = 0.0f;
+    ks[NB * STR + x] = 0.0f;
+  }
+#pragma unroll 4
   for (int x = tid; x < NB * D; x += 256) {
     const int t = x / D, d = x - t * D;
     const bool in = t0 + t < a.positions;
@@ -109,15 +117,13 @@ __global__ void __launch_bounds__(256) wkv_coef_k(KxWkvArgs a) {
   __syncthreads();
   float acc[NB] = {};  // of token j - d
   for (int c = sl; c < D; c += 16) {
-    const float r = rs[j * STR + c];
-    float p = r;
-    acc[0] = __builtin_fmaf(r * a.u[h * D + c], ks[j * STR + c], acc[0]);
+    float p = rs[j * STR + c];
+    const float *k = ks + j * STR + c, *wt = ws + j * STR + c;
+    acc[0] = __builtin_fmaf(p * a.u[h * D + c], k[0], acc[0]);
 #pragma unroll
     for (int d = 1; d < NB; ++d) {
-      const int i = max(j - d, 0);
-      const float k = d <= j ? ks[i * STR + c] : 0.0f;
-      acc[d] = __builtin_fmaf(p, k, acc[d]);
-      p *= ws[i * STR + c];
+      acc[d] = __builtin_fmaf(p, k[-d * STR], acc[d]);
+      p *= wt[-d * STR];
     }
   }
   float mine = 0.0f;  // lane s holds i = s
@@ -131,18 +137,26 @@ __global__ void __launch_bounds__(256) wkv_coef_k(KxWkvArgs a) {
     if (j - d == sl) mine = v;
   }
   w.inner[(((size_t)b * a.s.heads + h) * padded + t0 + j) * NB + sl] = mine;
-  for (int c = tid; c < D; c += 256) {
-    float p = 1.0f;
+  constexpr int Q = 4, PER = NB / Q;  // a thread has a quarter of the block's tokens of one channel
+  for (int x = tid; x < Q * D; x += 256) {
+    const int quarter = x / D, c = x - quarter * D, first = quarter * PER;
+    float dec[NB], p = 1.0f, s = 1.0f;
+#pragma unroll
+    for (int t = 0; t < NB; ++t) dec[t] = ws[t * STR + c];
+#pragma unroll
     for (int t = 0; t < NB; ++t) {
+      p *= t < first ? dec[t] : 1.0f;
+      s *= t >= first + PER ? dec[t] : 1.0f;
+    }
+#pragma unroll
+    for (int y = 0; y < PER; ++y) {
+      const int t = first + y, u = first + PER - 1 - y;
       if (t0 + t < a.positions) w.q[((size_t)(t0 + t) * a.batch + b) * HD + h * D + c] = rs[t * STR + c] * p;
+      if (t0 + u < a.positions) w.k[((size_t)(t0 + u) * a.batch + b) * HD + h * D + c] = ks[u * STR + c] * s;
       p *= ws[t * STR + c];
+      s *= ws[u * STR + c];
     }
-    w.total[(((size_t)b * a.s.heads + h) * (padded / NB) + blockIdx.x) * D + c] = p;
-    p = 1.0f;
-    for (int t = NB - 1; t >= 0; --t) {
-      if (t0 + t < a.positions) w.k[((size_t)(t0 + t) * a.batch + b) * HD + h * D + c] = ks[t * STR + c] * p;
-      p *= ws[t * STR + c];
-    }
+    if (quarter == Q - 1) w.total[(((size_t)b * a.s.heads + h) * (padded / NB) + blockIdx.x) * D + c] = p;
   }
 }
 
@@ -179,10 +193,10 @@ int kx_wkv_launch(bool f32, const KxWkvArgs &a, hipStream_t st) {
   g.out_ld = hd;
   int rc = kx_linear_launch(f32, g, a.rows, st);
   if (rc) return rc;
-  const size_t lds = (size_t)3 * NB * (s.dim + 16) * 4;
+  const size_t lds = coef_lds(s.dim);
   static std::atomic<bool> attr{false};
   if (!attr) {
-    KX_HIP(hipFuncSetAttribute((const void *)wkv_coef_k, hipFuncAttributeMaxDynamicSharedMemorySize, 3 * NB * (KX_SCAN_MAX_DIM + 16) * 4));
+    KX_HIP(hipFuncSetAttribute((const void *)wkv_coef_k, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024));
     attr = true;
   }
   hipLaunchKernelGGL(wkv_coef_k, dim3(padded / NB, s.heads, a.batch), dim3(256), lds, st, a);
